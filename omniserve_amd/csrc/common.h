@@ -114,15 +114,13 @@ __device__ __forceinline__ half_t silu_mul_h(half_t a, half_t b) {
 //   * |x| <= max|x| makes |x * q| <= 127 (1 + 2^-23): the saturation can never fire, no clamp;
 //   * NaN products (NaN or inf inputs: inf * 0) keep a NaN through the add, and every NaN this path can produce --
 //     the default NaN and widened fp16 payloads -- has a zero low byte: code 0, which is cvt.rni.sat's NaN -> 0.
-typedef float v2f_t __attribute__((ext_vector_type(2)));
 __device__ __forceinline__ float quant_multiplier(float amax) {
   // 127 / amax; an all-zero row (amax = 0: the reference divides by zero, then 0 * inf = NaN -> code 0) gets 0 so that the
   // products are 0 -> code 0 without going through NaN
   return amax == 0.0f ? 0.0f : 127.0f / amax;
 }
 // f32(x) * q in ONE instruction (v_fma_mix_f32 widens the fp16 operand itself; fma(x, q, +0) is the once-rounded product,
-// i.e. v_cvt_f32_f16 + v_mul_f32) -- hipcc emits shift + convert + multiply; and the packed f32 add as written (left to
-// itself the backend splits most of the pairs again).
+// i.e. v_cvt_f32_f16 + v_mul_f32) -- hipcc emits shift + convert + multiply.
 __device__ __forceinline__ float mul_f16lo_f32(uint32_t h2, float q) {
   float r;
   asm("v_fma_mix_f32 %0, %1, %2, 0 op_sel_hi:[1,0,0]" : "=v"(r) : "v"(h2), "v"(q));
@@ -133,22 +131,14 @@ __device__ __forceinline__ float mul_f16hi_f32(uint32_t h2, float q) {
   asm("v_fma_mix_f32 %0, %1, %2, 0 op_sel:[1,0,0] op_sel_hi:[1,0,0]" : "=v"(r) : "v"(h2), "v"(q));
   return r;
 }
-// (64-bit integer operands: with <2 x float> asm outputs hipcc 7.2 read element 0 for both elements of the result)
-__device__ __forceinline__ uint64_t pk_add_f32_bits(uint64_t a, uint64_t b) {
-  uint64_t r;
-  asm("v_pk_add_f32 %0, %1, %2" : "=v"(r) : "v"(a), "v"(b));
-  return r;
-}
 __device__ __forceinline__ uint32_t quant4_f16(uint32_t h01, uint32_t h23, float q) {
-  constexpr uint64_t magic = 0x4B4000004B400000ull;       // {1.5 * 2^23, 1.5 * 2^23}
-  auto pair = [](float lo, float hi) -> uint64_t {
-    return ((uint64_t)__builtin_bit_cast(uint32_t, hi) << 32) | __builtin_bit_cast(uint32_t, lo);
-  };
-  const uint64_t pa = pk_add_f32_bits(pair(mul_f16lo_f32(h01, q), mul_f16hi_f32(h01, q)), magic);
-  const uint64_t pb = pk_add_f32_bits(pair(mul_f16lo_f32(h23, q), mul_f16hi_f32(h23, q)), magic);
+  constexpr float magic = 12582912.0f;                    // 1.5 * 2^23
+  auto bits = [](float v) -> uint32_t { return __builtin_bit_cast(uint32_t, v); };
+  const uint32_t a0 = bits(mul_f16lo_f32(h01, q) + magic), a1 = bits(mul_f16hi_f32(h01, q) + magic);
+  const uint32_t b0 = bits(mul_f16lo_f32(h23, q) + magic), b1 = bits(mul_f16hi_f32(h23, q) + magic);
   // v_perm_b32(S0, S1, sel): selector byte 0-3 -> byte of S1, 4-7 -> byte of S0, 0x0c -> 0x00
-  const uint32_t lo = __builtin_amdgcn_perm((uint32_t)(pa >> 32), (uint32_t)pa, 0x0c0c0400u);
-  const uint32_t hi = __builtin_amdgcn_perm((uint32_t)(pb >> 32), (uint32_t)pb, 0x04000c0cu);
+  const uint32_t lo = __builtin_amdgcn_perm(a1, a0, 0x0c0c0400u);
+  const uint32_t hi = __builtin_amdgcn_perm(b1, b0, 0x04000c0cu);
   return lo | hi;
 }
 

@@ -408,7 +408,7 @@ __global__ __launch_bounds__(256, 2) void w4a8_gemm_exact_kernel(GemmArgs p) {
     return;
   }
   // The lane's 16 channels are the same for every row block: their scales are converted once (32 registers the K loop
-  // no longer needs); the arithmetic runs on float pairs (v_pk_mul_f32 / v_pk_add_f32: the reference's three products and one
+  // no longer needs); the arithmetic runs on float pairs (the reference's three products and one
   // difference, each rounded to f32 -- -ffp-contract=off) and the pair is made opaque before the fp16 conversion: hipcc
   // otherwise folds `(half)(f32 * f32)` into v_fma_mixlo_f16 -- ONE rounding to fp16 where the reference rounds to f32 first --
   // and a handful of outputs per million differ by one fp16 ulp (caught by the cross-build checksum of tools/gemm_ab.py).

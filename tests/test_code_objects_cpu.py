@@ -27,7 +27,7 @@ SPILL_ALLOWED = [
     (r"w4a8_gemv_kernelILi4ELi0ELb0ELi4E", 6),      # per-channel 64-row tile, 4 K parts, in-kernel epilogue
     (r"w4a8_gemv_kernelILi4ELi1ELb[01]ELi4E", 8),   # per-group 64-row tile, 4 K parts
     (r"w4a8_gemv_kernelILi1ELi1ELb1ELi[24]ELb[01]ELi1ELi0ELb1E", 8),   # per-group fp16-input GEMV (level 3 on g128 layers)
-    (r"w4a8_gemm_kernelILi8ELi2ELi4ELb[01]ELb0E", 7),   # W8A8 ragged-shape 128-row tile: ring of 2 measured 5 - 7 % faster than the
+    (r"w4a8_gemm_kernelILi8ELi2ELi4ELb[01]ELb0E", 8),   # W8A8 ragged-shape 128-row tile: ring of 2 measured 5 - 7 % faster than the
                                                         # spill-free ring of 1 (tools/ragged_gemm_ab.py)
 ]
 

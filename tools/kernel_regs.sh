@@ -3,7 +3,7 @@
 # usage: tools/kernel_regs.sh qgemm_chn.hip midm [extra hipcc flags]
 cd "$(dirname "$0")/../omniserve_amd/csrc" || exit 1
 src=$1; pat=$2; shift 2
-/opt/rocm/bin/hipcc --offload-arch=gfx950 -O3 -std=c++17 -fPIC -ffp-contract=off -I. -I../../include "$@" -c "$src" -o /tmp/kr_$$.o \
+/opt/rocm/bin/hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 -std=c++17 -fPIC -ffp-contract=off -I. -I../../include "$@" -c "$src" -o /tmp/kr_$$.o \
   -Rpass-analysis=kernel-resource-usage 2>&1 | awk -v pat="$pat" '
   /Function Name:/ { name=$0; sub(/.*Function Name: /,"",name); sub(/ \[.*/,"",name); keep = (name ~ pat) }
   keep && /VGPRs:/ && !/Spill/ { v=$0; sub(/.*VGPRs: /,"",v); sub(/ \[.*/,"",v) }
