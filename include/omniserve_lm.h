@@ -1,0 +1,95 @@
+/* C ABI of the serving engine's layer kernels (libomniserve_lm_bf16.so, libomniserve_lm_f32.so: the same entry points for one
+ * element type each).  Device pointers, sizes, strides in elements, a hipStream_t; every call only enqueues (no allocation, no
+ * synchronisation).  Returns 0, -22 (arguments) or -5 (launch).  "elem" is the library's element type.
+ *
+ * Conventions of the callers' data: inner sizes are padded with zeros to multiples of 64 (model width, feed-forward, and per
+ * head to 64 / 128 / 256), so that no kernel guards a k loop; statistics take the real size as an argument. */
+#pragma once
+#include <stdint.h>
+
+#ifdef __cplusplus
+extern "C" {
+#endif
+
+#define LM_ABI_VERSION 1
+#define LM_NORM_LAYER 0
+#define LM_NORM_RMS 1
+#define LM_EPI_ELEM 0
+#define LM_EPI_F32 1
+#define LM_EPI_GLU 2
+#define LM_ACT_NONE 0
+#define LM_ACT_SILU 1
+#define LM_ATTN_ROWS 128 /* query rows of one lm_attn_prefill tile */
+
+int lm_abi_version(void);
+int lm_elem_bytes(void);
+
+/* Residual stream x (f32) and the norms around it, one token per row:
+ *   x = embed[tokens]  (tokens given)      y = sublayer output, or the weighted sum of its expert rows (top > 0)
+ *   x += norm(y; post_w, post_b)           (post_w null: x += y;  y null: nothing added)
+ *   h = norm(x; next_w, next_b)            (next_w null: no h)
+ * kind: LM_NORM_LAYER / LM_NORM_RMS over the first n columns.  Expert rows: (token, choice) pair t * top + k of y, weight
+ * pair_w of the same index; shared != 0: row pairs0 + t is added with weight one.  rows: row r of h belongs to token rows[r]. */
+int lm_residual_norm(float* x, int64_t ldx, const int* tokens, const void* embed, const void* y, int64_t ldy, const float* pair_w,
+                     int top, int pairs0, int shared, const float* post_w, const float* post_b, const float* next_w,
+                     const float* next_b, void* h, int64_t ldh, const int* rows, int n_rows, int n, int kind, int store_x, float eps,
+                     void* stream);
+
+/* out = rms_norm(o) * w * sigmoid(gate); n real columns of cols */
+int lm_gated_rms(void* out, int64_t ldo, const void* o, int64_t ldi, const void* gate, int64_t ldg, const float* w, int rows, int cols,
+                 int n, float eps, void* stream);
+
+/* Rows q [H][dk] k [G][dk] v [G][dv]: q, k turned in place / into the cache, v mixed ((1 - lambda) v + lambda v_first) into the
+ * cache.  freq: rotation per position of each of the `half` pairs.  slot = page * 64 + offset, < 0: not stored. */
+int lm_rope_append(void* qkv, int64_t ld, const void* v_first, int64_t ldv, float lambda, const float* freq, int half, const int* pos,
+                   const int* slot, void* kc, void* vc, int tokens, int H, int G, int dk, int dv, void* stream);
+
+/* Causal sliding-window attention of prompt portions over the paged cache (pages of 64 tokens, [page][G][64][dk | dv]).
+ * entry [.][4]: first token, tokens, position of the first token, block table row; tiles [n_tiles][2]: entry, first row. */
+int lm_attn_prefill(const void* q, int64_t ldq, const void* kc, const void* vc, const int* bt, int bt_stride, const int* entry,
+                    const int* tiles, int n_tiles, const void* gate, int64_t ldg, void* o, int64_t ldo, float scale, int window, int H,
+                    int G, int dk, int dv, void* stream);
+
+/* One token per sequence: rotation + value mixing + append + attention + gate.  part: f32 [B][H][nsplit][dv + 2] for nsplit > 1. */
+int lm_attn_decode(const void* qkv, int64_t ld, const void* v_first, int64_t ldv, float lambda, const float* freq, int half,
+                   const int* pos, const int* slot, void* kc, void* vc, const int* bt, int bt_stride, const void* gate, int64_t ldg,
+                   void* o, int64_t ldo, float* part, int nsplit, float scale, int window, int B, int H, int G, int dk, int dv,
+                   void* stream);
+
+/* Decayed linear attention; rows q [H][dk] k [H][dk] v [H][dv], `act` applied to all three.  seg [.][8]: first token, tokens,
+ * slot, starts from zero, index in its entry, segments of the entry, 0, 0; all but an entry's last have seg_len tokens.
+ * multi: some entry has several segments (seg_state: f32 [segments][H][dk][dv]). */
+int lm_linear_prefill(const void* x, int64_t ld, void* o, int64_t ldo, float* state, float* seg_state, const int* seg, int segments,
+                      int seg_len, int multi, const float* log2_decay, int H, int dk, int dv, int act, void* stream);
+int lm_linear_decode(const void* x, int64_t ld, void* o, int64_t ldo, float* state, const int* slot, const int* pos,
+                     const float* log2_decay, int B, int H, int dk, int dv, int act, void* stream);
+
+/* z [tokens][ldz] f32 router logits -> wts [tokens][top], off [experts + 1], perm [tokens * top] (pairs sorted by expert);
+ * with tiles: [max][2] (expert, first place) of every 128-row tile, n_tiles [1]. */
+int64_t lm_route_scratch_words(int tokens, int experts, int top);
+int lm_route_max_tiles(int tokens, int experts, int top);
+int lm_route(const float* z, int64_t ldz, const float* bias, int tokens, int experts, int top, float* wts, int* off, int* perm,
+             int* tiles, int* n_tiles, int* scratch_i32, void* stream);
+
+/* y = x w^T for one or many matrices w [groups][n][k].  perm null: one group, rows_a rows.  Else group g has the places
+ * off[g] .. off[g + 1] of perm; a place's y row is perm[place], its x row perm[place] / x_div.  b (optional): one more matrix over
+ * rows 0 .. rows_b - 1 of its own x and y.  epi: LM_EPI_ELEM, LM_EPI_F32 (times scale), LM_EPI_GLU (rows of w in
+ * alternating blocks of 16 gate / 16 up channels; y has n / 2 columns: silu(gate) * up). */
+typedef struct {
+  const void* w;
+  const void* x;
+  int64_t ldx;
+  void* y;
+  int64_t ldy;
+  int n, k;
+} LmGemmPart;
+int lm_gemm_rows(const LmGemmPart* a, const LmGemmPart* b, int groups, const int* perm, const int* off, int rows_a, int rows_b,
+                 int x_div, int max_rows, float scale, int epi, void* stream);
+int lm_gemm_tiles(const LmGemmPart* a, const LmGemmPart* b, int groups, const int* perm, const int* off, const int* tiles,
+                  const int* n_tiles, int max_tiles, int rows_a, int rows_b, int x_div, float scale, int epi, void* stream);
+
+int lm_argmax(int64_t* out, const float* z, int64_t ld, int rows, int n, void* stream);
+
+#ifdef __cplusplus
+}
+#endif

@@ -1,0 +1,172 @@
+// Expert choice and the order of the grouped products: per token the `top` largest router logits (ties: the lower expert) and
+// their softmax; then the (token, choice) pairs sorted by expert -- off[experts + 1], perm[pairs] -- and the 128-row tiles of
+// every expert for lm_gemm_tiles.
+#include "lm_common.h"
+#include "omniserve_lm.h"
+
+namespace lm {
+
+constexpr int MAX_EXPERTS = 512, MAX_TOP = 16;
+
+// one wave per token; lane l looks at experts l, l + 64, ...; every lane ends up with the same choices
+__device__ __forceinline__ void choose(const float* z, const float* bias, int experts, int top, int lane, int* ids, float* wts) {
+  float v[MAX_EXPERTS / 64];
+#pragma unroll
+  for (int i = 0; i < MAX_EXPERTS / 64; ++i) {
+    const int e = lane + 64 * i;
+    v[i] = e < experts ? z[e] + (bias ? bias[e] : 0.f) : -INFINITY;
+  }
+  float best0 = 0.f, sum = 0.f, mine = 0.f;
+  int my_id = 0;
+  for (int k = 0; k < top; ++k) {
+    float b = -INFINITY;
+    int at = 0x7fffffff;
+#pragma unroll
+    for (int i = 0; i < MAX_EXPERTS / 64; ++i)
+      if (v[i] > b) { b = v[i]; at = lane + 64 * i; }
+#pragma unroll
+    for (int m = 32; m > 0; m >>= 1) {
+      const float ob = __shfl_xor(b, m, 64);
+      const int oa = __shfl_xor(at, m, 64);
+      if (ob > b || (ob == b && oa < at)) { b = ob; at = oa; }
+    }
+    if (at >= experts) at = k;        // only NaN logits get here: any in-range expert
+    if (k == 0) best0 = b;
+    const float ex = __expf(b - best0);
+    sum += ex;
+    if (lane == k) { mine = ex; my_id = at; }
+#pragma unroll
+    for (int i = 0; i < MAX_EXPERTS / 64; ++i)
+      if (at == lane + 64 * i) v[i] = -INFINITY;
+  }
+  if (lane < top) { ids[lane] = my_id; wts[lane] = mine / sum; }
+}
+
+// everything for up to 64 tokens in one workgroup
+__global__ __launch_bounds__(1024) void route_small_kernel(const float* z, int64_t ldz, const float* bias, int tokens, int experts,
+                                                           int top, float* wts, int* off, int* perm) {
+  __shared__ int ids[64 * MAX_TOP], count[MAX_EXPERTS], start[MAX_EXPERTS + 1];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, pairs = tokens * top;
+  for (int e = tid; e < experts; e += 1024) count[e] = 0;
+  for (int t = wave; t < tokens; t += 16) choose(z + (int64_t)t * ldz, bias, experts, top, lane, ids + t * top, wts + (int64_t)t * top);
+  __syncthreads();
+  int rank = 0, e = 0;
+  if (tid < pairs) {
+    e = ids[tid];
+    rank = atomicAdd(&count[e], 1);
+  }
+  __syncthreads();
+  if (wave == 0) {                   // prefix sum of the counts, 64 experts at a time
+    int base = 0;
+    for (int e0 = 0; e0 < experts; e0 += 64) {
+      const int c = e0 + lane < experts ? count[e0 + lane] : 0;
+      int s = c;
+#pragma unroll
+      for (int m = 1; m < 64; m <<= 1) {
+        const int o = __shfl_up(s, m, 64);
+        if (lane >= m) s += o;
+      }
+      if (e0 + lane < experts) start[e0 + lane] = base + s - c;
+      base += __shfl(s, 63, 64);
+    }
+    if (lane == 0) start[experts] = base;
+  }
+  __syncthreads();
+  if (tid < pairs) perm[start[e] + rank] = tid;
+  for (int i = tid; i <= experts; i += 1024) off[i] = start[i];
+}
+
+// many tokens: choices with their rank inside the expert (counts aggregated per workgroup before the global atomics) ...
+__global__ __launch_bounds__(256) void route_choose_kernel(const float* z, int64_t ldz, const float* bias, int tokens, int experts,
+                                                           int top, float* wts, int* ids, int* rank, int* count) {
+  __shared__ int hist[MAX_EXPERTS], base[MAX_EXPERTS], lid[64 * MAX_TOP];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, t0 = blockIdx.x * 64, n = min(64, tokens - t0);
+  for (int e = tid; e < experts; e += 256) hist[e] = 0;
+  for (int t = wave; t < n; t += 4)
+    choose(z + (int64_t)(t0 + t) * ldz, bias, experts, top, lane, lid + t * top, wts + (int64_t)(t0 + t) * top);
+  __syncthreads();
+  int r[64 * MAX_TOP / 256];
+#pragma unroll
+  for (int i = 0; i < 64 * MAX_TOP / 256; ++i)
+    if (tid + 256 * i < n * top) r[i] = atomicAdd(&hist[lid[tid + 256 * i]], 1);
+  __syncthreads();
+  for (int e = tid; e < experts; e += 256) base[e] = hist[e] ? atomicAdd(&count[e], hist[e]) : 0;
+  __syncthreads();
+#pragma unroll
+  for (int i = 0; i < 64 * MAX_TOP / 256; ++i) {
+    const int k = tid + 256 * i;
+    if (k < n * top) {
+      ids[(int64_t)t0 * top + k] = lid[k];
+      rank[(int64_t)t0 * top + k] = base[lid[k]] + r[i];
+    }
+  }
+}
+
+// ... offsets and row tiles ...
+__global__ __launch_bounds__(512) void route_offsets_kernel(const int* count, int experts, int* off, int* tiles, int* n_tiles) {
+  __shared__ int s_off[MAX_EXPERTS], s_tile[MAX_EXPERTS];
+  const int e = threadIdx.x, c = e < experts ? count[e] : 0, nt = (c + 127) / 128;
+  s_off[e] = c;
+  s_tile[e] = nt;
+  __syncthreads();
+  for (int m = 1; m < 512; m <<= 1) {
+    const int a = e >= m ? s_off[e - m] : 0, b = e >= m ? s_tile[e - m] : 0;
+    __syncthreads();
+    s_off[e] += a;
+    s_tile[e] += b;
+    __syncthreads();
+  }
+  if (e < experts) {
+    const int o = s_off[e] - c, t = s_tile[e] - nt;
+    off[e] = o;
+    for (int i = 0; i < nt; ++i) {
+      tiles[2 * (t + i)] = e;
+      tiles[2 * (t + i) + 1] = o + 128 * i;
+    }
+    if (e == experts - 1) {
+      off[experts] = s_off[e];
+      n_tiles[0] = s_tile[e];
+    }
+  }
+}
+
+// ... and the pairs in their places
+__global__ __launch_bounds__(256) void route_scatter_kernel(const int* ids, const int* rank, const int* off, int pairs, int* perm) {
+  const int i = blockIdx.x * 256 + threadIdx.x;
+  if (i < pairs) perm[off[ids[i]] + rank[i]] = i;
+}
+
+__global__ __launch_bounds__(512) void clear_kernel(int* p, int n) {
+  if ((int)threadIdx.x < n) p[threadIdx.x] = 0;
+}
+
+}  // namespace lm
+
+using namespace lm;
+
+// scratch_i32: lm_route_scratch_words(tokens, experts, top) words (more than 64 tokens only)
+extern "C" int64_t lm_route_scratch_words(int tokens, int experts, int top) { return MAX_EXPERTS + 2 * (int64_t)tokens * top; }
+extern "C" int lm_route_max_tiles(int tokens, int experts, int top) {
+  const int64_t pairs = (int64_t)tokens * top;
+  return (int)(pairs / 128 + (pairs < experts ? pairs : experts));
+}
+
+extern "C" int lm_route(const float* z, int64_t ldz, const float* bias, int tokens, int experts, int top, float* wts, int* off,
+                        int* perm, int* tiles, int* n_tiles, int* scratch_i32, void* stream) {
+  if (tokens <= 0 || experts <= 0 || experts > MAX_EXPERTS || top <= 0 || top > MAX_TOP || top > experts || ldz < experts ||
+      (int64_t)tokens * top > (1 << 28))
+    return LM_EINVAL;
+  hipStream_t s = (hipStream_t)stream;
+  if (tokens <= 64 && !tiles) {
+    hipLaunchKernelGGL(route_small_kernel, dim3(1), dim3(1024), 0, s, z, ldz, bias, tokens, experts, top, wts, off, perm);
+    return launch_status();
+  }
+  if (!tiles || !n_tiles || !scratch_i32) return LM_EINVAL;
+  const int pairs = tokens * top;
+  int *count = scratch_i32, *ids = count + MAX_EXPERTS, *rank = ids + pairs;
+  hipLaunchKernelGGL(clear_kernel, dim3(1), dim3(512), 0, s, count, MAX_EXPERTS);
+  hipLaunchKernelGGL(route_choose_kernel, dim3((tokens + 63) / 64), dim3(256), 0, s, z, ldz, bias, tokens, experts, top, wts, ids, rank, count);
+  hipLaunchKernelGGL(route_offsets_kernel, dim3(1), dim3(512), 0, s, count, experts, off, tiles, n_tiles);
+  hipLaunchKernelGGL(route_scatter_kernel, dim3((pairs + 255) / 256), dim3(256), 0, s, ids, rank, off, pairs, perm);
+  return launch_status();
+}

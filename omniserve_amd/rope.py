@@ -4,11 +4,35 @@ table[pos, i] = (cos, sin)(pos * scale / base**(2i/dim)) in float32, i < dim/2 -
 reference evaluates on the device (common/decoderMaskedMultiheadAttentionUtils.h:1147-1152).
 Building it once on the host (numpy float32) makes the RoPE bit-reproducible and removes
 powf/sincosf from the bandwidth-bound kernels.
+
+`inverse_frequencies` is what the engine's layers use instead: they turn by position * frequency inside the kernel.
 """
 from __future__ import annotations
 
+import math
+
 import numpy as np
 import torch
+
+
+def inverse_frequencies(dims: int, base: float, scaling=None) -> list:
+    """Rotation per position of the dims // 2 pairs (float64), base**(-2i/dims).
+
+    scaling {factor, low, high, original}: frequencies of wavelengths below original / high stay, those above original / low are
+    divided by factor, in between the two are blended linearly in original / wavelength."""
+    out = []
+    for i in range(dims // 2):
+        f = float(base) ** (-2.0 * i / dims)
+        if scaling:
+            turns = scaling["original"] * f / (2.0 * math.pi)          # within the original context
+            if turns < scaling["low"]:
+                f /= scaling["factor"]
+            elif turns <= scaling["high"]:
+                s = (turns - scaling["low"]) / (scaling["high"] - scaling["low"])
+                f = (1.0 - s) * f / scaling["factor"] + s * f
+        out.append(f)
+    return out
+
 
 _cache = {}
 _retired = []     # superseded tables stay allocated: captured HIP graphs hold their raw pointers
