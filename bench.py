@@ -672,6 +672,20 @@ def _parallelism(args, world):
             if args.tp_mode else "replicas x%d (no collective)" % world)
 
 
+def design_bench(args):
+    if not torch.cuda.is_available():
+        raise SystemExit("bench.py needs an MI355X (no CPU fallback: the HIP path is the product)")
+    from omniserve_amd.engine import benchmark
+    device = torch.device("cuda:0")
+    torch.cuda.set_device(device)
+    sizes = tuple(benchmark.SIZES) if args.design == "all" else (args.design,)
+    res = benchmark.run(device, sizes, llama=not args.no_extras)
+    first = res[sizes[0]]["bobavik_bf16"]["decode_bs16"]
+    print(json.dumps({"metric": "decode tokens/s, Bobavik %s, bs 16, 1024 cached tokens" % sizes[0], "value": first["tokens_per_s"],
+                      "unit": "tokens/s", "n_gpus": 1, "ms_per_step": first["ms_per_step"], "higher_is_better": True,
+                      "vs_baseline": None, "dtype": "bf16", "data": "synthetic (random weights and tokens)", "designs": res}), flush=True)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1, help="N > 1 without a launcher (WORLD_SIZE unset): bench.py starts the N ranks "
@@ -697,7 +711,12 @@ def main():
                          "two ranks on one GPU only -- no multi-GPU box was available to its author)")
     ap.add_argument("--tp", action="store_true", help="(default with N > 1; kept for older command lines) shard ONE model over "
                     "the N GPUs: Megatron TP, fp16 sum all-reduce after o_proj / down_proj inside the step; strong scaling")
+    ap.add_argument("--design", nargs="?", const="all", default=None, metavar="SIZE",
+                    help="instead of the workload above: prefill and decode throughput of the Bobavik design at real layer sizes beside "
+                         "the W4A8KV4 Llama of equal size (omniserve_amd/engine/benchmark.py; SIZE: all, 4096 or 2048)")
     args = ap.parse_args()
+    if args.design:
+        return design_bench(args)
 
     if "WORLD_SIZE" not in os.environ and args.gpus > 1:
         # no launcher around us: become one.  One process per GPU under torch.distributed.run, same arguments.

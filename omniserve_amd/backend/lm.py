@@ -21,7 +21,8 @@ EPI_ELEM, EPI_F32, EPI_GLU = 0, 1, 2
 ABI = 1
 ATTN_ROWS = 128          # query rows of one prefill tile
 PAGE = 64                # tokens per cache page
-ROWS_MAX = 64            # most rows the weight-streaming products take
+ROWS_MAX = 64            # up to here a step's products stream the weights
+NARROW = 128             # products of so few channels do for any number of rows
 
 
 class _Part(_c.Structure):
@@ -127,7 +128,7 @@ class LmOps:
             return torch.mm(x, w.t(), out=out)
         part = _Part(_p(w), _p(x), _ld(x), _p(out), _ld(out), n, w.shape[1])
         epi = EPI_F32 if out_f32 else EPI_ELEM
-        if T <= ROWS_MAX:
+        if T <= ROWS_MAX or n <= NARROW:
             self._call("lm_gemm_rows", _c.byref(part), None, 1, None, None, T, 0, 1, T, scale, epi)
         else:
             self._call("lm_gemm_tiles", _c.byref(part), None, 1, None, None, None, None, 0, T, 0, 1, scale, epi)

@@ -191,22 +191,32 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(DecodeArgs p) {
   }
 }
 
-__global__ __launch_bounds__(64) void attn_merge_kernel(const float* part, int nsplit, const int* pos, const elem_t* gate, int64_t ldg,
-                                                        elem_t* o, int64_t ldo, int H, int dv) {
-  const int b = blockIdx.x, h = blockIdx.y;
+// one workgroup per (sequence, head); at most 64 parts: lane s of every wave holds the maximum and sum of part s
+__global__ __launch_bounds__(256) void attn_merge_kernel(const float* part, int nsplit, const int* pos, const elem_t* gate, int64_t ldg,
+                                                         elem_t* o, int64_t ldo, int H, int dv) {
+  const int b = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63;
   if (pos[b] < 0) return;
   const float* q = part + ((int64_t)b * H + h) * nsplit * (dv + 2);
-  float m = NEG;
-  for (int s = 0; s < nsplit; ++s) m = fmaxf(m, q[s * (dv + 2)]);
-  float l = 0.f;
-  for (int s = 0; s < nsplit; ++s) l += __builtin_amdgcn_exp2f(q[s * (dv + 2)] - m) * q[s * (dv + 2) + 1];
-  for (int d = threadIdx.x; d < dv; d += 64) {
-    float y = 0.f;
-    for (int s = 0; s < nsplit; ++s) y += __builtin_amdgcn_exp2f(q[s * (dv + 2)] - m) * q[s * (dv + 2) + 2 + d];
-    y /= l;
-    if (gate) y *= sigmoid((float)gate[(int64_t)b * ldg + (int64_t)h * dv + d]);
-    o[(int64_t)b * ldo + (int64_t)h * dv + d] = (elem_t)y;
+  const int64_t step = dv + 2;
+  const bool in = lane < nsplit;
+  const float ms = in ? q[lane * step] : NEG, ls = in ? q[lane * step + 1] : 0.f;
+  float m = ms;
+#pragma unroll
+  for (int k = 32; k > 0; k >>= 1) m = fmaxf(m, __shfl_xor(m, k, 64));
+  const float f = __builtin_amdgcn_exp2f(ms - m), inv = 1.0f / wave_sum(f * ls);
+  const int d = threadIdx.x;
+  float y = 0.f;
+  for (int s0 = 0; s0 < nsplit; s0 += 8) {
+    float v[8];
+#pragma unroll
+    for (int s = 0; s < 8; ++s) v[s] = d < dv && s0 + s < nsplit ? q[(s0 + s) * step + 2 + d] : 0.f;
+#pragma unroll
+    for (int s = 0; s < 8; ++s) y += __shfl(f, s0 + s, 64) * v[s];
   }
+  if (d >= dv) return;
+  y *= inv;
+  if (gate) y *= sigmoid((float)gate[(int64_t)b * ldg + (int64_t)h * dv + d]);
+  o[(int64_t)b * ldo + (int64_t)h * dv + d] = (elem_t)y;
 }
 
 template <int DK, int DV>
@@ -214,7 +224,7 @@ static int launch(const DecodeArgs& a, int B, hipStream_t s) {
   const int gs = a.H / a.G, hb = (gs + 15) / 16;
   hipLaunchKernelGGL((attn_decode_kernel<DK, DV>), dim3(B, a.G * hb, a.nsplit), dim3(256), 0, s, a);
   if (a.nsplit > 1)
-    hipLaunchKernelGGL(attn_merge_kernel, dim3(B, a.H), dim3(64), 0, s, a.part, a.nsplit, a.pos, a.gate, a.ldg, a.o, a.ldo, a.H, DV);
+    hipLaunchKernelGGL(attn_merge_kernel, dim3(B, a.H), dim3(256), 0, s, a.part, a.nsplit, a.pos, a.gate, a.ldg, a.o, a.ldo, a.H, DV);
   return launch_status();
 }
 
@@ -227,7 +237,7 @@ extern "C" int lm_attn_decode(const void* qkv, int64_t ld, const void* v_first, 
                               int64_t ldg, void* o, int64_t ldo, float* part, int nsplit, float scale, int window, int B, int H, int G,
                               int dk, int dv, void* stream) {
   if (B <= 0 || G <= 0 || H % G || !(scale > 0.f) || window <= 0 || half < 0 || 2 * half > dk || nsplit <= 0 || (nsplit > 1 && !part) ||
-      ld % FR || ldv % FR || ldo % 4 || ldg % 4 || nsplit > 1024)
+      ld % FR || ldv % FR || ldo % 4 || ldg % 4 || nsplit > 64)
     return LM_EINVAL;
   DecodeArgs a{(const elem_t*)qkv, ld, (const elem_t*)v_first, ldv, lambda, freq, half, pos, slot, (elem_t*)kc, (elem_t*)vc, bt, bt_stride,
                (const elem_t*)gate, ldg, (elem_t*)o, ldo, part, scale * 1.4426950408889634f, window, H, G, nsplit};

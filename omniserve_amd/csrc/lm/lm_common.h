@@ -80,8 +80,8 @@ __device__ __forceinline__ void split_quad(f32x4 x, quad_t (&q)[NOPND]) {
   if constexpr (SPLIT) q[NOPND - 1] = to_quad(x - from_quad(q[0]));
 }
 
-__device__ __forceinline__ float sigmoid(float z) { return 1.0f / (1.0f + __expf(-z)); }
-__device__ __forceinline__ float silu(float z) { return z / (1.0f + __expf(-z)); }
+__device__ __forceinline__ float sigmoid(float z) { return __builtin_amdgcn_rcpf(1.0f + __expf(-z)); }      // (rcp: within an ulp)
+__device__ __forceinline__ float silu(float z) { return z * sigmoid(z); }
 
 // lam^n for n >= 0, from log2(lam)
 __device__ __forceinline__ float power(float log2_lam, int n) { return n == 0 ? 1.0f : __builtin_amdgcn_exp2f((float)n * log2_lam); }

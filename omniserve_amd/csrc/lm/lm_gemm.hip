@@ -44,22 +44,25 @@ __device__ __forceinline__ void store4(const Part& pt, int64_t row, int c, f32x4
   }
 }
 
-// NR 16-channel blocks x MB 16-row blocks per workgroup, KW waves split K
-template <int NR, int MB, int KW, int EPI>
-__global__ __launch_bounds__(64 * KW) void gemm_rows_kernel(GemmArgs p) {
-  constexpr int U = NR * MB >= 8 ? 4 : 8;       // k-steps in flight
-  __shared__ __attribute__((aligned(16))) float red[KW][16 * MB][16 * NR + 4];
+// A workgroup owns 16 NR NW channels: NW groups of waves take NR 16-channel blocks each (they read the same rows of x, out of the
+// CU's L1), the KW waves of a group split K and meet in LDS.  16 MB rows at a time; blockIdx.z takes every gridDim.z-th such part.
+template <int NR, int MB, int NW, int KW, int EPI>
+__global__ __launch_bounds__(64 * NW * KW) void gemm_rows_kernel(GemmArgs p) {
+  constexpr int U = NR * MB >= 2 ? 4 : 8;       // k-steps requested together
+  __shared__ __attribute__((aligned(16))) float red_all[NW][KW][16 * MB][16 * NR + 4];
   const int g = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l15 = lane & 15, l4 = lane >> 4;
+  const int nw = wave / KW, kw = wave % KW, gt = tid - nw * 64 * KW;      // group, K part, thread within the group
+  float(*red)[16 * MB][16 * NR + 4] = red_all[nw];
   const bool is_b = g >= p.groups;
   const Part& pt = is_b ? p.b : p.a;
-  const int n0 = blockIdx.x * 16 * NR;
-  if (n0 >= pt.n) return;
+  if ((int)blockIdx.x * 16 * NR * NW >= pt.n) return;
+  const int n0 = (blockIdx.x * NW + nw) * 16 * NR;
   int first = 0, rows = is_b ? p.rows_b : p.rows_a;
   const int* perm = is_b ? nullptr : p.perm;
   if (perm) { first = p.off[g]; rows = p.off[g + 1] - first; }
   if (rows <= 0) return;
   const elem_t* w = pt.w + (is_b ? 0 : (int64_t)g * pt.n * pt.k);
-  const int steps = pt.k / KSTEP, s0 = steps * wave / KW, s1 = steps * (wave + 1) / KW;
+  const int steps = pt.k / KSTEP, s0 = steps * kw / KW, s1 = steps * (kw + 1) / KW;
   const elem_t* wp[NR];
 #pragma unroll
   for (int r = 0; r < NR; ++r) {
@@ -67,7 +70,7 @@ __global__ __launch_bounds__(64 * KW) void gemm_rows_kernel(GemmArgs p) {
     wp[r] = w + (int64_t)(c < pt.n ? c : pt.n - 1) * pt.k + FR * l4;
   }
   const int div = is_b ? 1 : p.x_div;
-  for (int m0 = 0; m0 < rows; m0 += 16 * MB) {
+  for (int m0 = 16 * MB * blockIdx.z; m0 < rows; m0 += 16 * MB * gridDim.z) {
     const elem_t* xp[MB];
 #pragma unroll
     for (int m = 0; m < MB; ++m) {
@@ -81,13 +84,14 @@ __global__ __launch_bounds__(64 * KW) void gemm_rows_kernel(GemmArgs p) {
     for (int r = 0; r < NR; ++r)
 #pragma unroll
       for (int m = 0; m < MB; ++m) acc[r][m] = zero4();
-    int s = s0;
-    for (; s + U <= s1; s += U) {
-      frag_t wf[NR][U];
+    frag_t wf[NR][U], wn[NR][U];
+    auto request = [&](frag_t (&f)[NR][U], int s) {
 #pragma unroll
       for (int u = 0; u < U; ++u)
 #pragma unroll
-        for (int r = 0; r < NR; ++r) wf[r][u] = __builtin_nontemporal_load((const frag_t*)(wp[r] + (int64_t)(s + u) * KSTEP));
+        for (int r = 0; r < NR; ++r) f[r][u] = __builtin_nontemporal_load((const frag_t*)(wp[r] + (int64_t)(s + u) * KSTEP));
+    };
+    auto multiply = [&](frag_t (&f)[NR][U], int s) {
 #pragma unroll
       for (int m = 0; m < MB; ++m) {
         if (m < mb) {
@@ -97,30 +101,41 @@ __global__ __launch_bounds__(64 * KW) void gemm_rows_kernel(GemmArgs p) {
 #pragma unroll
           for (int u = 0; u < U; ++u)
 #pragma unroll
-            for (int r = 0; r < NR; ++r) acc[r][m] = mma(wf[r][u], xf[u], acc[r][m]);
+            for (int r = 0; r < NR; ++r) acc[r][m] = mma(f[r][u], xf[u], acc[r][m]);
         }
       }
+    };
+    int s = s0;
+    if (s + U <= s1) request(wf, s);
+    while (s + U <= s1) {              // the next U steps are on their way while these multiply
+      if (s + 2 * U <= s1) request(wn, s + U);
+      multiply(wf, s);
+      s += U;
+      if (s + U > s1) break;
+      if (s + 2 * U <= s1) request(wf, s + U);
+      multiply(wn, s);
+      s += U;
     }
     for (; s < s1; ++s) {
-      frag_t wf[NR];
+      frag_t w1[NR];
 #pragma unroll
-      for (int r = 0; r < NR; ++r) wf[r] = *(const frag_t*)(wp[r] + (int64_t)s * KSTEP);
+      for (int r = 0; r < NR; ++r) w1[r] = *(const frag_t*)(wp[r] + (int64_t)s * KSTEP);
 #pragma unroll
       for (int m = 0; m < MB; ++m) {
         if (m < mb) {
           const frag_t xf = *(const frag_t*)(xp[m] + (int64_t)s * KSTEP);
 #pragma unroll
-          for (int r = 0; r < NR; ++r) acc[r][m] = mma(wf[r], xf, acc[r][m]);
+          for (int r = 0; r < NR; ++r) acc[r][m] = mma(w1[r], xf, acc[r][m]);
         }
       }
     }
 #pragma unroll
     for (int r = 0; r < NR; ++r)
 #pragma unroll
-      for (int m = 0; m < MB; ++m) *(f32x4*)&red[wave][16 * m + l15][16 * r + 4 * l4] = acc[r][m];
+      for (int m = 0; m < MB; ++m) *(f32x4*)&red[kw][16 * m + l15][16 * r + 4 * l4] = acc[r][m];
     __syncthreads();
     constexpr int OB = EPI == LM_EPI_GLU ? NR / 2 : NR;      // 16-channel blocks of the result
-    for (int i = tid; i < 16 * MB * OB * 4; i += 64 * KW) {
+    for (int i = gt; i < 16 * MB * OB * 4; i += 64 * KW) {
       const int m = i / (OB * 4), q = i - m * (OB * 4), blk = q >> 2, c4 = 4 * (q & 3);
       const int sb = EPI == LM_EPI_GLU ? 2 * blk : blk;
       if (m0 + m >= rows) continue;
@@ -223,29 +238,60 @@ __global__ __launch_bounds__(256, 2) void gemm_tiles_kernel(GemmArgs p, int mt_a
     step(wt0, xt0, wt1, xt1, k0 + TK);
     if (k0 + TK < pt.k) step(wt1, xt1, wt0, xt0, k0 + 2 * TK);
   }
+  if constexpr (EPI == LM_EPI_F32) {
 #pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const int m = wm + 16 * j + l15;
-    if (m >= rows) continue;
-    const int64_t row = perm ? perm[first + m] : first + m;
-    if constexpr (EPI == LM_EPI_GLU) {
-#pragma unroll
-      for (int i = 0; i < 4; i += 2) {
-        const int c = (n0 + wn + 16 * i) / 2 + 4 * l4;
-        if (c < pt.n / 2) store4<EPI>(pt, row, c, acc[i][j], acc[i + 1][j], 1.f);
-      }
-    } else {
+    for (int j = 0; j < 4; ++j) {
+      const int m = wm + 16 * j + l15;
+      if (m >= rows) continue;
+      const int64_t row = perm ? perm[first + m] : first + m;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int c = n0 + wn + 16 * i + 4 * l4;
         if (c < pt.n) store4<EPI>(pt, row, c, acc[i][j], zero4(), p.scale);
       }
     }
+  } else {
+    // through LDS, so that a row leaves in whole 16-byte pieces of neighbouring lanes; a wave handles its own 64 rows x (64 or
+    // 32) channels in two halves of 32 rows (all tiles have been read: the last step ended with a barrier)
+    constexpr int OC = EPI == LM_EPI_GLU ? 32 : 64, PITCH = OC * (int)sizeof(elem_t) + 16, PPR = OC / FR;
+    uint8_t* buf = wave == 0 ? wt0 : wave == 1 ? wt1 : wave == 2 ? xt0 : xt1;
+    static_assert(32 * PITCH <= TN * TROWB, "a wave's half fits its buffer");
+#pragma unroll
+    for (int half = 0; half < 2; ++half) {
+#pragma unroll
+      for (int jj = 0; jj < 2; ++jj) {
+        const int j = 2 * half + jj;
+#pragma unroll
+        for (int i = 0; i < 4; i += EPI == LM_EPI_GLU ? 2 : 1) {
+          f32x4 v = acc[i][j];
+          int c = 16 * i;
+          if constexpr (EPI == LM_EPI_GLU) {
+            c = 8 * i;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = silu(v[e]) * acc[i + 1][j][e];
+          }
+          *(quad_t*)(buf + (16 * jj + l15) * PITCH + (c + 4 * l4) * (int)sizeof(elem_t)) = to_quad(v);
+        }
+      }
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+      __builtin_amdgcn_wave_barrier();
+#pragma unroll
+      for (int i = 0; i < 32 * PPR / 64; ++i) {
+        const int pc = 64 * i + lane, r = pc / PPR, q = pc % PPR;
+        const int m = wm + 32 * half + r, c = (EPI == LM_EPI_GLU ? (n0 + wn) / 2 : n0 + wn) + q * FR;
+        if (m < rows && c < (EPI == LM_EPI_GLU ? pt.n / 2 : pt.n)) {
+          const int64_t row = perm ? perm[first + m] : first + m;
+          *(frag_t*)((elem_t*)pt.y + row * pt.ldy + c) = *(const frag_t*)(buf + r * PITCH + q * 16);
+        }
+      }
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+      __builtin_amdgcn_wave_barrier();
+    }
   }
 }
 
 static int check_part(const Part& p, int epi) {
-  if (!p.w || !p.x || !p.y || p.n <= 0 || p.k <= 0 || p.k % 64 || p.n % 4 || p.ldx < p.k || p.ldx % FR || p.ldy % 4) return LM_EINVAL;
+  if (!p.w || !p.x || !p.y || p.n <= 0 || p.k <= 0 || p.k % 64 || p.n % 16 || p.ldx < p.k || p.ldx % FR || p.ldy % FR) return LM_EINVAL;
   if (epi == LM_EPI_GLU && p.n % 32) return LM_EINVAL;
   return LM_OK;
 }
@@ -264,14 +310,32 @@ static int fill(GemmArgs& a, const LmGemmPart* pa, const LmGemmPart* pb, int gro
   return LM_OK;
 }
 
-template <int NR, int EPI>
+template <int NR, int NW, int KW, int EPI>
 static int launch_rows(const GemmArgs& a, int max_rows, int has_b, hipStream_t s) {
   const int n = has_b && a.b.n > a.a.n ? a.b.n : a.a.n;
-  const dim3 grid((n + 16 * NR - 1) / (16 * NR), a.groups + has_b);
-  if (max_rows <= 16) hipLaunchKernelGGL((gemm_rows_kernel<NR, 1, 8, EPI>), grid, dim3(512), 0, s, a);
-  else if (max_rows <= 32) hipLaunchKernelGGL((gemm_rows_kernel<NR, 2, 8, EPI>), grid, dim3(512), 0, s, a);
-  else hipLaunchKernelGGL((gemm_rows_kernel<NR, 4, 4, EPI>), grid, dim3(256), 0, s, a);
+  const int mb = max_rows <= 16 ? 1 : max_rows <= 32 ? 2 : 4;
+  const dim3 grid((n + 16 * NR * NW - 1) / (16 * NR * NW), a.groups + has_b, a.perm ? 1 : (max_rows + 16 * mb - 1) / (16 * mb));
+  const dim3 block(64 * NW * KW);
+  if (mb == 1) hipLaunchKernelGGL((gemm_rows_kernel<NR, 1, NW, KW, EPI>), grid, block, 0, s, a);
+  else if (mb == 2) hipLaunchKernelGGL((gemm_rows_kernel<NR, 2, NW, KW, EPI>), grid, block, 0, s, a);
+  else hipLaunchKernelGGL((gemm_rows_kernel<NR, 4, NW, KW, EPI>), grid, block, 0, s, a);
   return launch_status();
+}
+
+// Channels per workgroup: as many as still leave a workgroup for every CU (fewer reads of x).  A product of few channels over
+// many rows (the router of a prompt) has its workgroups along the rows instead.
+template <int EPI>
+static int plan_rows(const GemmArgs& a, int max_rows, int has_b, hipStream_t s) {
+  const int64_t n = (int64_t)a.groups * a.a.n;
+  if constexpr (EPI == LM_EPI_GLU) {
+    return launch_rows<2, 1, 8, EPI>(a, max_rows, has_b, s);
+  } else {
+    if (max_rows > 64) return launch_rows<2, 1, 8, EPI>(a, max_rows, has_b, s);
+    if (n >= 128 * 256) return launch_rows<2, 4, 2, EPI>(a, max_rows, has_b, s);
+    if (n >= 64 * 240) return launch_rows<1, 4, 2, EPI>(a, max_rows, has_b, s);
+    if (n >= 32 * 240) return launch_rows<1, 2, 4, EPI>(a, max_rows, has_b, s);
+    return launch_rows<1, 1, 8, EPI>(a, max_rows, has_b, s);
+  }
 }
 
 }  // namespace lm
@@ -284,11 +348,8 @@ extern "C" int lm_gemm_rows(const LmGemmPart* pa, const LmGemmPart* pb, int grou
   if (fill(a, pa, pb, groups, perm, off, rows_a, rows_b, x_div, scale, epi) || max_rows <= 0) return LM_EINVAL;
   hipStream_t s = (hipStream_t)stream;
   const int has_b = pb && rows_b > 0;
-  // wide matrices: two 16-channel blocks per workgroup (half the activation reads); narrow ones: more workgroups
-  const bool wide = (int64_t)a.groups * a.a.n >= 32 * 768;
-  if (epi == LM_EPI_GLU) return launch_rows<2, LM_EPI_GLU>(a, max_rows, has_b, s);
-  if (epi == LM_EPI_F32) return wide ? launch_rows<2, LM_EPI_F32>(a, max_rows, has_b, s) : launch_rows<1, LM_EPI_F32>(a, max_rows, has_b, s);
-  return wide ? launch_rows<2, LM_EPI_ELEM>(a, max_rows, has_b, s) : launch_rows<1, LM_EPI_ELEM>(a, max_rows, has_b, s);
+  if (epi == LM_EPI_GLU) return plan_rows<LM_EPI_GLU>(a, max_rows, has_b, s);
+  return epi == LM_EPI_F32 ? plan_rows<LM_EPI_F32>(a, max_rows, has_b, s) : plan_rows<LM_EPI_ELEM>(a, max_rows, has_b, s);
 }
 
 extern "C" int lm_gemm_tiles(const LmGemmPart* pa, const LmGemmPart* pb, int groups, const int* perm, const int* off,

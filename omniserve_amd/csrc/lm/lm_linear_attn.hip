@@ -2,7 +2,7 @@
 //
 // Prompt portions, chunks of C tokens: with S the state before the chunk and i, j places in it (n of them)
 //     o_i = lam^(i+1) S^T q_i + sum_{j <= i} lam^(i-j) (q_i . k_j) v_j          S' = lam^n S + sum_j lam^(n-1-j) k_j v_j^T
-// A workgroup owns 64 value columns of one head and walks the chunks of one segment of a sequence; S stays in MFMA accumulators
+// A workgroup owns 64 or 128 value columns of one head and walks the chunks of one segment of a sequence; S stays in MFMA accumulators
 // (16 columns per wave).  Its accumulator layout is the quad layout of S^T as an operand, so the state never passes through LDS.
 // f32 factors (S, the decayed score matrix, the decayed values) enter the bf16 products as two bf16 operands each.
 // Long portions are cut into segments that run in parallel: a first pass forms what each segment adds to the state, the second
@@ -23,13 +23,14 @@ struct LinArgs {
   int H, dv, seg_len, act;
 };
 
-template <int DK>
+template <int DK, int NWV>
 struct LinGeom {
+  static constexpr int TH = 64 * NWV, DVB = 16 * NWV;                  // threads, value columns of a workgroup
   static constexpr int C = SPLIT ? 64 : 32;                            // tokens per chunk
-  static constexpr int KB = DK * (int)sizeof(elem_t), VB = 64 * (int)sizeof(elem_t);
+  static constexpr int KB = DK * (int)sizeof(elem_t), VB = DVB * (int)sizeof(elem_t);
   static constexpr int PB = C * (int)sizeof(elem_t) + 16;              // row of the score matrix
   static constexpr int Q0 = 0, K0 = C * KB, V0 = 2 * C * KB, P0 = V0 + C * VB, LDS = P0 + NOPND * C * PB;
-  static constexpr int NQ = C * KB / 4096, NV = C * VB / 4096;         // 16-byte loads per thread
+  static constexpr int NQ = C * KB / (16 * TH), NV = C * VB / (16 * TH);         // 16-byte loads per thread
 };
 
 constexpr int linear_waves_per_simd(int dk) { return SPLIT && dk <= 128 ? 2 : 1; }      // what the registers allow
@@ -42,16 +43,16 @@ __device__ __forceinline__ frag_t activate(frag_t v, int act) {
   return v;
 }
 
-template <int DK, bool OUTPUT>
-__global__ __launch_bounds__(256, linear_waves_per_simd(DK)) void linear_prefill_kernel(LinArgs p) {
-  typedef LinGeom<DK> Gm;
+template <int DK, int NWV, bool OUTPUT>
+__global__ __launch_bounds__(64 * NWV, linear_waves_per_simd(DK)) void linear_prefill_kernel(LinArgs p) {
+  typedef LinGeom<DK, NWV> Gm;
   typedef Tile<Gm::KB> KT;
   typedef Tile<Gm::VB> VT;
   constexpr int C = Gm::C, NS = DK / 16, NKF = DK / KSTEP, RT = C / 16;
   extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
   uint8_t *qt = lds + Gm::Q0, *kt = lds + Gm::K0, *vt = lds + Gm::V0, *pt = lds + Gm::P0;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l15 = lane & 15, l4 = lane >> 4;
-  const int sg = blockIdx.x, h = blockIdx.y, dv0 = 64 * blockIdx.z;
+  const int sg = blockIdx.x, h = blockIdx.y, dv0 = Gm::DVB * blockIdx.z;
   const int *sp = p.seg + 8 * sg;
   const int row0 = sp[0], count = sp[1], slot = sp[2], fresh = sp[3], idx = sp[4], nseg = sp[5];
   if (!OUTPUT && idx == nseg - 1) return;             // nothing follows the last segment
@@ -92,7 +93,7 @@ __global__ __launch_bounds__(256, linear_waves_per_simd(DK)) void linear_prefill
   auto fetch = [&](int c0) {
 #pragma unroll
     for (int i = 0; i < Gm::NQ; ++i) {
-      const int sl = 256 * i + tid, r = sl / KT::NS, s = sl % KT::NS;
+      const int sl = Gm::TH * i + tid, r = sl / KT::NS, s = sl % KT::NS;
       const bool in = c0 + r < count;
       const elem_t* a = src + (int64_t)(in ? c0 + r : 0) * p.ld + s * FR;
       if constexpr (OUTPUT) rq[i] = in ? *(const frag_t*)(a + qo) : frag_t{};
@@ -100,23 +101,33 @@ __global__ __launch_bounds__(256, linear_waves_per_simd(DK)) void linear_prefill
     }
 #pragma unroll
     for (int i = 0; i < Gm::NV; ++i) {
-      const int sl = 256 * i + tid, r = sl / VT::NS, s = sl % VT::NS;
+      const int sl = Gm::TH * i + tid, r = sl / VT::NS, s = sl % VT::NS;
       const bool in = c0 + r < count;
       rv[i] = in ? *(const frag_t*)(src + (int64_t)(c0 + r) * p.ld + vo + s * FR) : frag_t{};
     }
   };
+  // decay factors of a whole chunk
+  f32x4 wv[RT];                                        // of v_j in the new state
+  float wo[RT];                                        // of the state in row i
+#pragma unroll
+  for (int u = 0; u < RT; ++u) {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) wv[u][r] = power(ld, C - 1 - (16 * u + 4 * l4 + r));
+    wo[u] = power(ld, 16 * u + l15 + 1);
+  }
+  const float wc = power(ld, C), ld1 = power(ld, 1), ld2 = ld1 * ld1, ld3 = ld2 * ld1;
   fetch(0);
   for (int c0 = 0; c0 < count; c0 += C) {
     const int n = min(C, count - c0);
 #pragma unroll
     for (int i = 0; i < Gm::NQ; ++i) {
-      const int sl = 256 * i + tid, off = KT::slot(sl / KT::NS, sl % KT::NS);
+      const int sl = Gm::TH * i + tid, off = KT::slot(sl / KT::NS, sl % KT::NS);
       if constexpr (OUTPUT) *(frag_t*)(qt + off) = activate(rq[i], p.act);
       *(frag_t*)(kt + off) = activate(rk[i], p.act);
     }
 #pragma unroll
     for (int i = 0; i < Gm::NV; ++i) {
-      const int sl = 256 * i + tid;
+      const int sl = Gm::TH * i + tid;
       *(frag_t*)(vt + VT::slot(sl / VT::NS, sl % VT::NS)) = activate(rv[i], p.act);
     }
     __syncthreads();
@@ -125,28 +136,32 @@ __global__ __launch_bounds__(256, linear_waves_per_simd(DK)) void linear_prefill
 #pragma unroll
     for (int u = 0; u < RT; ++u) vq[u][0] = VT::column_quad(vt, 16 * u, wave, l15, l4);
     if constexpr (OUTPUT) {
-      // decayed scores, row block `wave`: transposed product, column = row i of the score matrix
-      if (wave < RT) {
-        const int i = 16 * wave + l15;
+      // decayed scores (transposed product: column = row i of the score matrix); blocks (row it, key u) of the lower triangle
+      // go round the waves.  The block right of an even diagonal block is read behind: zeros.
+      constexpr int BLOCKS = RT * RT;
 #pragma unroll
-        for (int u = 0; u < RT; ++u) {
-          if (u > (wave | 1)) continue;                // (the block right of an even diagonal block is read: zeros)
-          f32x4 s = zero4();
-          if (u <= wave) {
+      for (int bi = 0; bi < (BLOCKS + NWV - 1) / NWV; ++bi) {
+        const int it = wave % RT, u = bi * (NWV / RT > 0 ? NWV / RT : 1) + wave / RT;
+        if (it >= RT || u >= RT || u > (it | 1)) continue;
+        const int i = 16 * it + l15;
+        f32x4 s = zero4();
+        if (u <= it) {
 #pragma unroll
-            for (int k = 0; k < NKF; ++k) s = mma(KT::frag(kt, 16 * u + l15, 4 * k + l4), KT::frag(qt, i, 4 * k + l4), s);
+          for (int k = 0; k < NKF; ++k) s = mma(KT::frag(kt, 16 * u + l15, 4 * k + l4), KT::frag(qt, i, 4 * k + l4), s);
+          const int d0 = i - (16 * u + 4 * l4);       // distance of the lane's first key
+          if (u < it) {
+            const float f = power(ld, d0 - 3);
+            s *= (f32x4){f * ld3, f * ld2, f * ld1, f};
+          } else {
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-              const int d = i - (16 * u + 4 * l4 + r);
-              s[r] = d >= 0 ? s[r] * power(ld, d) : 0.f;
-            }
+            for (int r = 0; r < 4; ++r) s[r] = d0 >= r ? s[r] * power(ld, d0 - r) : 0.f;
           }
-          quad_t q[NOPND];
-          split_quad(s, q);
-#pragma unroll
-          for (int o = 0; o < NOPND; ++o)
-            *(quad_t*)(pt + (o * C + i) * Gm::PB + (16 * u + 4 * l4) * (int)sizeof(elem_t)) = q[o];
         }
+        quad_t q[NOPND];
+        split_quad(s, q);
+#pragma unroll
+        for (int o = 0; o < NOPND; ++o)
+          *(quad_t*)(pt + (o * C + i) * Gm::PB + (16 * u + 4 * l4) * (int)sizeof(elem_t)) = q[o];
       }
       // what the state in front of the chunk contributes: O^T = S^T Q^T, rows of this wave's 16 columns
       f32x4 out[RT];
@@ -165,7 +180,7 @@ __global__ __launch_bounds__(256, linear_waves_per_simd(DK)) void linear_prefill
         }
       }
 #pragma unroll
-      for (int it = 0; it < RT; ++it) out[it] *= power(ld, 16 * it + l15 + 1);
+      for (int it = 0; it < RT; ++it) out[it] *= wo[it];
       __syncthreads();
 #pragma unroll
       for (int it = 0; it < RT; ++it) {
@@ -185,18 +200,23 @@ __global__ __launch_bounds__(256, linear_waves_per_simd(DK)) void linear_prefill
       }
     }
     // S <- lam^n S + K^T (lam^(n-1-j) v_j)
-    const float fn = power(ld, n);
+    const float fn = n == C ? wc : power(ld, n);
 #pragma unroll
     for (int t = 0; t < NS; ++t) S[t] *= fn;
 #pragma unroll
     for (int kk = 0; kk < RT / 2; ++kk) {
       quad_t b0[NOPND], b1[NOPND];
       f32x4 x0 = from_quad(vq[2 * kk][0]), x1 = from_quad(vq[2 * kk + 1][0]);
+      if (n == C) {
+        x0 *= wv[2 * kk];
+        x1 *= wv[2 * kk + 1];
+      } else {
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int j = 32 * kk + 4 * l4 + r;            // (places from n on hold zeros)
-        x0[r] *= power(ld, max(n - 1 - j, 0));
-        x1[r] *= power(ld, max(n - 1 - j - 16, 0));
+        for (int r = 0; r < 4; ++r) {
+          const int j = 32 * kk + 4 * l4 + r;          // (places from n on hold zeros)
+          x0[r] *= power(ld, max(n - 1 - j, 0));
+          x1[r] *= power(ld, max(n - 1 - j - 16, 0));
+        }
       }
       split_quad(x0, b0);
       split_quad(x1, b1);
@@ -268,19 +288,28 @@ __global__ __launch_bounds__(256) void linear_decode_kernel(const elem_t* x, int
   }
 }
 
-template <int DK>
+template <int DK, int NWV>
 static int launch(const LinArgs& a, int segments, int multi, hipStream_t s) {
-  constexpr size_t lds = LinGeom<DK>::LDS;
-  const dim3 grid(segments, a.H, a.dv / 64);
+  constexpr size_t lds = LinGeom<DK, NWV>::LDS;
+  const dim3 grid(segments, a.H, a.dv / (16 * NWV)), block(64 * NWV);
   if (multi) {
-    auto k = linear_prefill_kernel<DK, false>;
+    auto k = linear_prefill_kernel<DK, NWV, false>;
     if (allow_lds(k, lds)) return LM_EINVAL;
-    hipLaunchKernelGGL(k, grid, dim3(256), lds, s, a);
+    hipLaunchKernelGGL(k, grid, block, lds, s, a);
   }
-  auto k = linear_prefill_kernel<DK, true>;
+  auto k = linear_prefill_kernel<DK, NWV, true>;
   if (allow_lds(k, lds)) return LM_EINVAL;
-  hipLaunchKernelGGL(k, grid, dim3(256), lds, s, a);
+  hipLaunchKernelGGL(k, grid, block, lds, s, a);
   return launch_status();
+}
+
+// 128 value columns share one staging of q and k where the registers allow
+template <int DK>
+static int plan(const LinArgs& a, int segments, int multi, hipStream_t s) {
+  if constexpr (SPLIT && DK <= 128) {
+    if (a.dv % 128 == 0) return launch<DK, 8>(a, segments, multi, s);
+  }
+  return launch<DK, 4>(a, segments, multi, s);
 }
 
 }  // namespace lm
@@ -293,9 +322,9 @@ extern "C" int lm_linear_prefill(const void* x, int64_t ld, void* o, int64_t ldo
   if (segments <= 0 || H <= 0 || dv % 64 || seg_len % 64 || seg_len <= 0 || (multi && !seg_state) || ld % FR || ldo % 4) return LM_EINVAL;
   LinArgs a{(const elem_t*)x, ld, (elem_t*)o, ldo, state, seg_state, seg, log2_decay, H, dv, seg_len, act};
   hipStream_t s = (hipStream_t)stream;
-  if (dk == 64) return launch<64>(a, segments, multi, s);
-  if (dk == 128) return launch<128>(a, segments, multi, s);
-  if (dk == 256) return launch<256>(a, segments, multi, s);
+  if (dk == 64) return plan<64>(a, segments, multi, s);
+  if (dk == 128) return plan<128>(a, segments, multi, s);
+  if (dk == 256) return plan<256>(a, segments, multi, s);
   return LM_EINVAL;
 }
 

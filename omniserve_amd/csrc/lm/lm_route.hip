@@ -7,12 +7,14 @@
 namespace lm {
 
 constexpr int MAX_EXPERTS = 512, MAX_TOP = 16;
+constexpr int CHOOSE_TOKENS = 16;      // tokens per workgroup of route_choose_kernel
 
-// one wave per token; lane l looks at experts l, l + 64, ...; every lane ends up with the same choices
+// one wave per token; lane l looks at its EPL experts l, l + 64, ...; every lane ends up with the same choices
+template <int EPL>
 __device__ __forceinline__ void choose(const float* z, const float* bias, int experts, int top, int lane, int* ids, float* wts) {
-  float v[MAX_EXPERTS / 64];
+  float v[EPL];
 #pragma unroll
-  for (int i = 0; i < MAX_EXPERTS / 64; ++i) {
+  for (int i = 0; i < EPL; ++i) {
     const int e = lane + 64 * i;
     v[i] = e < experts ? z[e] + (bias ? bias[e] : 0.f) : -INFINITY;
   }
@@ -22,7 +24,7 @@ __device__ __forceinline__ void choose(const float* z, const float* bias, int ex
     float b = -INFINITY;
     int at = 0x7fffffff;
 #pragma unroll
-    for (int i = 0; i < MAX_EXPERTS / 64; ++i)
+    for (int i = 0; i < EPL; ++i)
       if (v[i] > b) { b = v[i]; at = lane + 64 * i; }
 #pragma unroll
     for (int m = 32; m > 0; m >>= 1) {
@@ -36,19 +38,20 @@ __device__ __forceinline__ void choose(const float* z, const float* bias, int ex
     sum += ex;
     if (lane == k) { mine = ex; my_id = at; }
 #pragma unroll
-    for (int i = 0; i < MAX_EXPERTS / 64; ++i)
+    for (int i = 0; i < EPL; ++i)
       if (at == lane + 64 * i) v[i] = -INFINITY;
   }
   if (lane < top) { ids[lane] = my_id; wts[lane] = mine / sum; }
 }
 
 // everything for up to 64 tokens in one workgroup
+template <int EPL>
 __global__ __launch_bounds__(1024) void route_small_kernel(const float* z, int64_t ldz, const float* bias, int tokens, int experts,
                                                            int top, float* wts, int* off, int* perm) {
   __shared__ int ids[64 * MAX_TOP], count[MAX_EXPERTS], start[MAX_EXPERTS + 1];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, pairs = tokens * top;
   for (int e = tid; e < experts; e += 1024) count[e] = 0;
-  for (int t = wave; t < tokens; t += 16) choose(z + (int64_t)t * ldz, bias, experts, top, lane, ids + t * top, wts + (int64_t)t * top);
+  for (int t = wave; t < tokens; t += 16) choose<EPL>(z + (int64_t)t * ldz, bias, experts, top, lane, ids + t * top, wts + (int64_t)t * top);
   __syncthreads();
   int rank = 0, e = 0;
   if (tid < pairs) {
@@ -77,23 +80,24 @@ __global__ __launch_bounds__(1024) void route_small_kernel(const float* z, int64
 }
 
 // many tokens: choices with their rank inside the expert (counts aggregated per workgroup before the global atomics) ...
+template <int EPL>
 __global__ __launch_bounds__(256) void route_choose_kernel(const float* z, int64_t ldz, const float* bias, int tokens, int experts,
                                                            int top, float* wts, int* ids, int* rank, int* count) {
-  __shared__ int hist[MAX_EXPERTS], base[MAX_EXPERTS], lid[64 * MAX_TOP];
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, t0 = blockIdx.x * 64, n = min(64, tokens - t0);
+  __shared__ int hist[MAX_EXPERTS], base[MAX_EXPERTS], lid[CHOOSE_TOKENS * MAX_TOP];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, t0 = blockIdx.x * CHOOSE_TOKENS, n = min(CHOOSE_TOKENS, tokens - t0);
   for (int e = tid; e < experts; e += 256) hist[e] = 0;
   for (int t = wave; t < n; t += 4)
-    choose(z + (int64_t)(t0 + t) * ldz, bias, experts, top, lane, lid + t * top, wts + (int64_t)(t0 + t) * top);
+    choose<EPL>(z + (int64_t)(t0 + t) * ldz, bias, experts, top, lane, lid + t * top, wts + (int64_t)(t0 + t) * top);
   __syncthreads();
-  int r[64 * MAX_TOP / 256];
+  int r[CHOOSE_TOKENS * MAX_TOP / 256];
 #pragma unroll
-  for (int i = 0; i < 64 * MAX_TOP / 256; ++i)
+  for (int i = 0; i < CHOOSE_TOKENS * MAX_TOP / 256; ++i)
     if (tid + 256 * i < n * top) r[i] = atomicAdd(&hist[lid[tid + 256 * i]], 1);
   __syncthreads();
   for (int e = tid; e < experts; e += 256) base[e] = hist[e] ? atomicAdd(&count[e], hist[e]) : 0;
   __syncthreads();
 #pragma unroll
-  for (int i = 0; i < 64 * MAX_TOP / 256; ++i) {
+  for (int i = 0; i < CHOOSE_TOKENS * MAX_TOP / 256; ++i) {
     const int k = tid + 256 * i;
     if (k < n * top) {
       ids[(int64_t)t0 * top + k] = lid[k];
@@ -158,14 +162,16 @@ extern "C" int lm_route(const float* z, int64_t ldz, const float* bias, int toke
     return LM_EINVAL;
   hipStream_t s = (hipStream_t)stream;
   if (tokens <= 64 && !tiles) {
-    hipLaunchKernelGGL(route_small_kernel, dim3(1), dim3(1024), 0, s, z, ldz, bias, tokens, experts, top, wts, off, perm);
+    auto k = experts <= 64 ? route_small_kernel<1> : experts <= 128 ? route_small_kernel<2> : route_small_kernel<MAX_EXPERTS / 64>;
+    hipLaunchKernelGGL(k, dim3(1), dim3(1024), 0, s, z, ldz, bias, tokens, experts, top, wts, off, perm);
     return launch_status();
   }
   if (!tiles || !n_tiles || !scratch_i32) return LM_EINVAL;
   const int pairs = tokens * top;
   int *count = scratch_i32, *ids = count + MAX_EXPERTS, *rank = ids + pairs;
   hipLaunchKernelGGL(clear_kernel, dim3(1), dim3(512), 0, s, count, MAX_EXPERTS);
-  hipLaunchKernelGGL(route_choose_kernel, dim3((tokens + 63) / 64), dim3(256), 0, s, z, ldz, bias, tokens, experts, top, wts, ids, rank, count);
+  auto k = experts <= 64 ? route_choose_kernel<1> : experts <= 128 ? route_choose_kernel<2> : route_choose_kernel<MAX_EXPERTS / 64>;
+  hipLaunchKernelGGL(k, dim3((tokens + CHOOSE_TOKENS - 1) / CHOOSE_TOKENS), dim3(256), 0, s, z, ldz, bias, tokens, experts, top, wts, ids, rank, count);
   hipLaunchKernelGGL(route_offsets_kernel, dim3(1), dim3(512), 0, s, count, experts, off, tiles, n_tiles);
   hipLaunchKernelGGL(route_scatter_kernel, dim3((pairs + 255) / 256), dim3(256), 0, s, ids, rank, off, pairs, perm);
   return launch_status();

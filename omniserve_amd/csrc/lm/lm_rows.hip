@@ -7,22 +7,26 @@ namespace lm {
 
 constexpr int ROW_THREADS = 256;
 
-struct Row {      // block-wide sums over ROW_THREADS
-  float* red;
+template <int TH>
+struct Row {      // workgroup-wide sums
+  float* red;     // [2][TH / 64]
   int phase = 0;
   __device__ __forceinline__ float sum(float v) {
     v = wave_sum(v);
-    float* r = red + 4 * (phase & 1);      // two areas in turn: one barrier per sum
+    float* r = red + TH / 64 * (phase & 1);      // two areas in turn: one barrier per sum
     ++phase;
     if ((threadIdx.x & 63) == 0) r[threadIdx.x >> 6] = v;
     __syncthreads();
-    return (r[0] + r[1]) + (r[2] + r[3]);
+    float t = 0.f;
+#pragma unroll
+    for (int i = 0; i < TH / 64; i += 4) t += (r[i] + r[i + 1]) + (r[i + 2] + r[i + 3]);
+    return t;
   }
 };
 
-// v (columns 4 * (256 i + tid) .. + 3, zero from n on) -> normalised in place; kind 0: layer norm, 1: RMS norm
-template <int NV>
-__device__ __forceinline__ void normalise(f32x4 (&v)[NV], Row& row, int n, int kind, float eps, const float* w, const float* b) {
+// v (columns 4 * (TH i + tid) .. + 3, zero from n on) -> normalised in place; kind 0: layer norm, 1: RMS norm
+template <int TH, int NV>
+__device__ __forceinline__ void normalise(f32x4 (&v)[NV], Row<TH>& row, int n, int kind, float eps, const float* w, const float* b) {
   float mean = 0.f;
   if (kind == LM_NORM_LAYER) {
     float s = 0.f;
@@ -33,7 +37,7 @@ __device__ __forceinline__ void normalise(f32x4 (&v)[NV], Row& row, int n, int k
   float ss = 0.f;
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
-    const int c = 4 * (ROW_THREADS * i + (int)threadIdx.x);
+    const int c = 4 * (TH * i + (int)threadIdx.x);
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       v[i][e] = c + e < n ? v[i][e] - mean : 0.f;
@@ -43,7 +47,7 @@ __device__ __forceinline__ void normalise(f32x4 (&v)[NV], Row& row, int n, int k
   const float r = 1.0f / sqrtf(row.sum(ss) / (float)n + eps);
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
-    const int c = 4 * (ROW_THREADS * i + (int)threadIdx.x);
+    const int c = 4 * (TH * i + (int)threadIdx.x);
     if (c >= n) continue;
     const f32x4 ww = *(const f32x4*)(w + c);
     f32x4 bb = zero4();
@@ -66,17 +70,17 @@ struct ResidualArgs {
   float eps;
 };
 
-template <int NV>
-__global__ __launch_bounds__(ROW_THREADS) void residual_norm_kernel(ResidualArgs p) {
-  __shared__ float red[8];
-  Row row{red};
+template <int TH, int NV>
+__global__ __launch_bounds__(TH) void residual_norm_kernel(ResidualArgs p) {
+  __shared__ float red[2 * TH / 64];
+  Row<TH> row{red};
   const int r = blockIdx.x, t = p.rows ? p.rows[r] : r, tid = threadIdx.x;
   f32x4 x[NV], y[NV];
   float* xr = p.x + (int64_t)t * p.ldx;
   const elem_t* er = p.tokens ? p.embed + (int64_t)p.tokens[t] * p.ldx : nullptr;
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
-    const int c = 4 * (ROW_THREADS * i + tid);
+    const int c = 4 * (TH * i + tid);
     x[i] = y[i] = zero4();
     if (c >= p.n) continue;
     x[i] = er ? from_quad(*(const quad_t*)(er + c)) : *(const f32x4*)(xr + c);
@@ -84,40 +88,51 @@ __global__ __launch_bounds__(ROW_THREADS) void residual_norm_kernel(ResidualArgs
   if (p.y) {
     if (p.top > 0) {      // weighted sum of the chosen experts' rows (+ the shared expert's)
       const int64_t p0 = (int64_t)t * p.top;
-      for (int k = 0; k < p.top; ++k) {
-        const float w = p.pair_w[p0 + k];
-        const elem_t* yr = p.y + (p0 + k) * p.ldy;
+      constexpr int B = NV >= 8 ? 1 : NV >= 4 ? 2 : 4;      // rows in flight
+      for (int k0 = 0; k0 < p.top; k0 += B) {
+        quad_t v[B][NV];
+        float w[B];
 #pragma unroll
-        for (int i = 0; i < NV; ++i) {
-          const int c = 4 * (ROW_THREADS * i + tid);
-          if (c < p.n) y[i] += w * from_quad(*(const quad_t*)(yr + c));
+        for (int b = 0; b < B; ++b) {
+          const int k = min(k0 + b, p.top - 1);
+          w[b] = k0 + b < p.top ? p.pair_w[p0 + k] : 0.f;
+          const elem_t* yr = p.y + (p0 + k) * p.ldy;
+#pragma unroll
+          for (int i = 0; i < NV; ++i) {
+            const int c = 4 * (TH * i + tid);
+            v[b][i] = c < p.n ? *(const quad_t*)(yr + c) : to_quad(zero4());
+          }
         }
+#pragma unroll
+        for (int b = 0; b < B; ++b)
+#pragma unroll
+          for (int i = 0; i < NV; ++i) y[i] += w[b] * from_quad(v[b][i]);
       }
     }
     if (p.top == 0 || p.shared) {
       const elem_t* yr = p.y + (int64_t)(p.top > 0 ? p.pairs0 + t : t) * p.ldy;
 #pragma unroll
       for (int i = 0; i < NV; ++i) {
-        const int c = 4 * (ROW_THREADS * i + tid);
+        const int c = 4 * (TH * i + tid);
         if (c < p.n) y[i] += from_quad(*(const quad_t*)(yr + c));
       }
     }
-    if (p.post_w) normalise<NV>(y, row, p.n, p.kind, p.eps, p.post_w, p.post_b);
+    if (p.post_w) normalise<TH, NV>(y, row, p.n, p.kind, p.eps, p.post_w, p.post_b);
 #pragma unroll
     for (int i = 0; i < NV; ++i) x[i] += y[i];
   }
   if (p.store_x) {
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-      const int c = 4 * (ROW_THREADS * i + tid);
+      const int c = 4 * (TH * i + tid);
       if (c < p.ldx) *(f32x4*)(xr + c) = x[i];
     }
   }
   if (!p.next_w) return;
-  normalise<NV>(x, row, p.n, p.kind, p.eps, p.next_w, p.next_b);
+  normalise<TH, NV>(x, row, p.n, p.kind, p.eps, p.next_w, p.next_b);
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
-    const int c = 4 * (ROW_THREADS * i + tid);
+    const int c = 4 * (TH * i + tid);
     if (c < p.ldh) *(quad_t*)(p.h + (int64_t)r * p.ldh + c) = to_quad(x[i]);
   }
 }
@@ -128,7 +143,7 @@ __global__ __launch_bounds__(ROW_THREADS) void gated_rms_kernel(elem_t* out, int
                                                                 const elem_t* gate, int64_t ldg, const float* w, int cols, int n,
                                                                 float eps) {
   __shared__ float red[8];
-  Row row{red};
+  Row<ROW_THREADS> row{red};
   const int t = blockIdx.x, tid = threadIdx.x;
   f32x4 v[NV];
   float ss = 0.f;
@@ -251,9 +266,13 @@ extern "C" int lm_residual_norm(float* x, int64_t ldx, const int* tokens, const 
                  next_b, (elem_t*)h, ldh, rows, n, kind, store_x, eps};
   hipStream_t s = (hipStream_t)stream;
   const int64_t cols = ldx > ldh ? ldx : ldh;
-#define LM_CASE(NV) \
-  if (cols <= 1024 * NV) { hipLaunchKernelGGL((residual_norm_kernel<NV>), dim3(n_rows), dim3(ROW_THREADS), 0, s, a); return launch_status(); }
-  LM_CASE(1) LM_CASE(2) LM_CASE(4) LM_CASE(8) LM_CASE(16)
+#define LM_CASE(TH, NV) \
+  if (cols <= 4 * TH * NV) { hipLaunchKernelGGL((residual_norm_kernel<TH, NV>), dim3(n_rows), dim3(TH), 0, s, a); return launch_status(); }
+  LM_CASE(256, 1)
+  if (n_rows <= 256) {      // latency: the whole workgroup on one piece of the row
+    LM_CASE(512, 1) LM_CASE(1024, 1) LM_CASE(1024, 2) LM_CASE(1024, 4)
+  }
+  LM_CASE(256, 2) LM_CASE(256, 4) LM_CASE(256, 8) LM_CASE(256, 16)
 #undef LM_CASE
   return LM_EINVAL;
 }

@@ -308,7 +308,7 @@ def check(got, want, dtype, what=""):
     if dtype == F32:
         assert e.max() < 1e-4, (what, int(e.argmax()), e.max())
     else:
-        assert np.median(e) < 0.03 and (e > 0.1).mean() < 0.05, (what, np.median(e), (e > 0.1).mean())
+        assert np.median(e) < 0.03 and (e > 0.1).sum() <= max(2, 0.05 * e.size), (what, np.median(e), (e > 0.1).mean())
 
 
 @pytest.mark.parametrize("dtype", DTYPES, ids=str)
