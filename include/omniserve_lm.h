@@ -11,7 +11,7 @@
 extern "C" {
 #endif
 
-#define LM_ABI_VERSION 1
+#define LM_ABI_VERSION 2
 #define LM_NORM_LAYER 0
 #define LM_NORM_RMS 1
 #define LM_EPI_ELEM 0
@@ -19,6 +19,7 @@ extern "C" {
 #define LM_EPI_GLU 2
 #define LM_ACT_NONE 0
 #define LM_ACT_SILU 1
+#define LM_TILE_ROWS 256 /* rows of one lm_gemm_tiles tile */
 #define LM_ATTN_ROWS 128 /* query rows of one lm_attn_prefill tile */
 
 int lm_abi_version(void);
@@ -65,11 +66,11 @@ int lm_linear_decode(const void* x, int64_t ld, void* o, int64_t ldo, float* sta
                      const float* log2_decay, int B, int H, int dk, int dv, int act, void* stream);
 
 /* z [tokens][ldz] f32 router logits -> wts [tokens][top], off [experts + 1], perm [tokens * top] (pairs sorted by expert);
- * with tiles: [max][2] (expert, first place) of every 128-row tile, n_tiles [1]. */
+ * with tiles: [lm_route_max_tiles][4] (expert, first place, rows, 0) of every row tile, rows = 0 past the last. */
 int64_t lm_route_scratch_words(int tokens, int experts, int top);
 int lm_route_max_tiles(int tokens, int experts, int top);
 int lm_route(const float* z, int64_t ldz, const float* bias, int tokens, int experts, int top, float* wts, int* off, int* perm,
-             int* tiles, int* n_tiles, int* scratch_i32, void* stream);
+             int* tiles, int* scratch_i32, void* stream);
 
 /* y = x w^T for one or many matrices w [groups][n][k].  perm null: one group, rows_a rows.  Else group g has the places
  * off[g] .. off[g + 1] of perm; a place's y row is perm[place], its x row perm[place] / x_div.  b (optional): one more matrix over
@@ -86,7 +87,7 @@ typedef struct {
 int lm_gemm_rows(const LmGemmPart* a, const LmGemmPart* b, int groups, const int* perm, const int* off, int rows_a, int rows_b,
                  int x_div, int max_rows, float scale, int epi, void* stream);
 int lm_gemm_tiles(const LmGemmPart* a, const LmGemmPart* b, int groups, const int* perm, const int* off, const int* tiles,
-                  const int* n_tiles, int max_tiles, int rows_a, int rows_b, int x_div, float scale, int epi, void* stream);
+                  int max_tiles, int rows_a, int rows_b, int x_div, float scale, int epi, void* stream);
 
 int lm_argmax(int64_t* out, const float* z, int64_t ld, int rows, int n, void* stream);
 

@@ -18,7 +18,7 @@ ELEM = {torch.bfloat16: "bf16", torch.float32: "f32"}
 NORM = {"layer": 0, "rms": 1}
 ACT = {None: 0, "silu": 1}
 EPI_ELEM, EPI_F32, EPI_GLU = 0, 1, 2
-ABI = 1
+ABI = 2
 ATTN_ROWS = 128          # query rows of one prefill tile
 PAGE = 64                # tokens per cache page
 ROWS_MAX = 64            # up to here a step's products stream the weights
@@ -43,9 +43,9 @@ PROTOTYPES = {
     "lm_linear_decode": (_i, [_vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _vp]),
     "lm_route_scratch_words": (_i64, [_i, _i, _i]),
     "lm_route_max_tiles": (_i, [_i, _i, _i]),
-    "lm_route": (_i, [_vp, _i64, _vp, _i, _i, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp]),
+    "lm_route": (_i, [_vp, _i64, _vp, _i, _i, _i, _vp, _vp, _vp, _vp, _vp, _vp]),
     "lm_gemm_rows": (_i, [_PP, _PP, _i, _vp, _vp, _i, _i, _i, _i, _f, _i, _vp]),
-    "lm_gemm_tiles": (_i, [_PP, _PP, _i, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _f, _i, _vp]),
+    "lm_gemm_tiles": (_i, [_PP, _PP, _i, _vp, _vp, _vp, _i, _i, _i, _i, _f, _i, _vp]),
     "lm_argmax": (_i, [_vp, _vp, _i64, _i, _i, _vp]),
 }
 
@@ -131,7 +131,7 @@ class LmOps:
         if T <= ROWS_MAX or n <= NARROW:
             self._call("lm_gemm_rows", _c.byref(part), None, 1, None, None, T, 0, 1, T, scale, epi)
         else:
-            self._call("lm_gemm_tiles", _c.byref(part), None, 1, None, None, None, None, 0, T, 0, 1, scale, epi)
+            self._call("lm_gemm_tiles", _c.byref(part), None, 1, None, None, None, 0, T, 0, 1, scale, epi)
         return out
 
     def route(self, z, bias, experts, top):
@@ -140,19 +140,18 @@ class LmOps:
         wts = torch.empty((T, top), dtype=torch.float32, device=dev)
         off = torch.empty((experts + 1,), dtype=torch.int32, device=dev)
         perm = torch.empty((T * top,), dtype=torch.int32, device=dev)
-        tiles = n_tiles = scratch = None
+        tiles = scratch = None
         max_tiles = 0
         if T > ROWS_MAX:
             max_tiles = self._h.lm_route_max_tiles(T, experts, top)
-            tiles = torch.empty((max_tiles, 2), dtype=torch.int32, device=dev)
-            n_tiles = torch.empty((1,), dtype=torch.int32, device=dev)
+            tiles = torch.empty((max_tiles, 4), dtype=torch.int32, device=dev)
             scratch = torch.empty((self._h.lm_route_scratch_words(T, experts, top),), dtype=torch.int32, device=dev)
-        self._call("lm_route", _p(z), _ld(z), _p(bias), T, experts, top, _p(wts), _p(off), _p(perm), _p(tiles), _p(n_tiles), _p(scratch))
-        return wts, (off, perm, tiles, n_tiles, max_tiles, top)
+        self._call("lm_route", _p(z), _ld(z), _p(bias), T, experts, top, _p(wts), _p(off), _p(perm), _p(tiles), _p(scratch))
+        return wts, (off, perm, tiles, max_tiles, top)
 
     def grouped(self, order, tokens, x, w, y, x_is_pairs, glu, extra=None):
         """Expert products: w [experts, n, k]; x rows per token or per (token, choice); extra = (x, w, y) of the shared expert."""
-        off, perm, tiles, n_tiles, max_tiles, top = order
+        off, perm, tiles, max_tiles, top = order
         a = _Part(_p(w), _p(x), _ld(x), _p(y), _ld(y), w.shape[1], w.shape[2])
         b = None
         if extra is not None:
@@ -162,8 +161,7 @@ class LmOps:
         if tiles is None:
             self._call("lm_gemm_rows", _c.byref(a), pb, w.shape[0], _p(perm), _p(off), 0, rb, div, tokens, 1.0, epi)
         else:
-            self._call("lm_gemm_tiles", _c.byref(a), pb, w.shape[0], _p(perm), _p(off), _p(tiles), _p(n_tiles), max_tiles, 0, rb, div, 1.0,
-                       epi)
+            self._call("lm_gemm_tiles", _c.byref(a), pb, w.shape[0], _p(perm), _p(off), _p(tiles), max_tiles, 0, rb, div, 1.0, epi)
 
 
 _ops = {}

@@ -102,15 +102,21 @@ __device__ __forceinline__ float column_sum(float v) {
   return v + __shfl_xor(v, 32, 64);
 }
 
-// LDS tile of rows of ROWB bytes in 16-byte slots, slot s of row r stored at s ^ swizzle(r): 16 rows read at one logical slot
-// (fragments) and 8 rows read at one 32-byte block (transposed quads) both fall into different banks.
+// LDS tile of rows of ROWB bytes in 16-byte slots, slot s of row r stored at s ^ swizzle(r).  A fragment read (ds_read_b128)
+// serves lanes {0-3, 12-15, 20-23, 24-27} and the like together, i.e. rows 0-3 and 12-15 at one slot with rows 4-11 at its
+// neighbour: the swizzles of rows 4-11 are closed under flipping the low bit, so 16 different places of a 256-byte line answer.
+// A transposed read serves 8 consecutive rows at one 32-byte block: their swizzles differ above the low bit.
 template <int ROWB>
 struct Tile {
   static constexpr int NS = ROWB / 16;
   static_assert(NS >= 8 && (NS & (NS - 1)) == 0, "row size");
   __device__ __forceinline__ static int swizzle(int row) {
-    if constexpr (NS == 8) return (((row >> 1) & 3) << 1) | ((row >> 3) & 1);
-    return ((row & 7) << 1) | ((row >> 3) & 1);
+    if constexpr (NS == 8) {         // neighbouring rows share a line
+      const int q = (row >> 1) & 7;
+      return (((q ^ ((q >> 1) & 2)) & 3) << 1) | (q >> 2);
+    }
+    const int r = row & 15;
+    return (((r ^ ((r >> 1) & 4)) & 7) << 1) | (r >> 3);
   }
   __device__ __forceinline__ static int slot(int row, int s) { return row * ROWB + ((s ^ swizzle(row)) << 4); }
   // element col of row, byte offset

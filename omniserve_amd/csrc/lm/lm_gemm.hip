@@ -3,7 +3,7 @@
 //
 //   lm_gemm_rows   few rows (decode): HBM bound.  A workgroup owns 16 or 32 channels of a group and streams their weights
 //                  once; its waves split K and meet in LDS.  Weights are the A operand straight from global memory.
-//   lm_gemm_tiles  many rows (prefill): MFMA bound.  128 x 128 tiles, both operands by LDS-DMA, double buffered.
+//   lm_gemm_tiles  many rows (prefill): MFMA bound.  256 x 128 tiles, both operands by LDS-DMA, two stages ahead.
 //
 // Epilogues: element type, f32 times a factor, or the gated unit silu(gate) * up of a matrix whose rows alternate in blocks of
 // 16 between gate and up channels (both halves of a pair then sit in the same lane).
@@ -26,7 +26,7 @@ struct GemmArgs {
   const int* off;             // [groups + 1] sorted places of each group
   int rows_a, rows_b;
   int x_div;                  // x row = y row / x_div (tokens of (token, choice) pairs)
-  const int* tiles; const int* n_tiles;   // lm_gemm_tiles with perm: (group, first place) of every 128-row tile
+  const int* tiles;           // lm_gemm_tiles with perm: (group, first place, rows, 0) of every row tile, rows 0: none
   float scale;
 };
 
@@ -44,25 +44,23 @@ __device__ __forceinline__ void store4(const Part& pt, int64_t row, int c, f32x4
   }
 }
 
-// A workgroup owns 16 NR NW channels: NW groups of waves take NR 16-channel blocks each (they read the same rows of x, out of the
-// CU's L1), the KW waves of a group split K and meet in LDS.  16 MB rows at a time; blockIdx.z takes every gridDim.z-th such part.
-template <int NR, int MB, int NW, int KW, int EPI>
-__global__ __launch_bounds__(64 * NW * KW) void gemm_rows_kernel(GemmArgs p) {
-  constexpr int U = NR * MB >= 2 ? 4 : 8;       // k-steps requested together
-  __shared__ __attribute__((aligned(16))) float red_all[NW][KW][16 * MB][16 * NR + 4];
+// A workgroup owns NR 16-channel blocks; its KW waves split K and meet in LDS.  16 MB rows at a time; blockIdx.z takes every
+// gridDim.z-th such part.
+template <int NR, int MB, int KW, int EPI>
+__global__ __launch_bounds__(64 * KW) void gemm_rows_kernel(GemmArgs p) {
+  constexpr int U = NR > 1 ? 4 : 8;             // k-steps of weights requested together (a multiple of 4: see xf)
+  __shared__ __attribute__((aligned(16))) float red[KW][16 * MB][16 * NR + 4];
   const int g = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l15 = lane & 15, l4 = lane >> 4;
-  const int nw = wave / KW, kw = wave % KW, gt = tid - nw * 64 * KW;      // group, K part, thread within the group
-  float(*red)[16 * MB][16 * NR + 4] = red_all[nw];
   const bool is_b = g >= p.groups;
   const Part& pt = is_b ? p.b : p.a;
-  if ((int)blockIdx.x * 16 * NR * NW >= pt.n) return;
-  const int n0 = (blockIdx.x * NW + nw) * 16 * NR;
+  const int n0 = blockIdx.x * 16 * NR;
+  if (n0 >= pt.n) return;
   int first = 0, rows = is_b ? p.rows_b : p.rows_a;
   const int* perm = is_b ? nullptr : p.perm;
   if (perm) { first = p.off[g]; rows = p.off[g + 1] - first; }
   if (rows <= 0) return;
   const elem_t* w = pt.w + (is_b ? 0 : (int64_t)g * pt.n * pt.k);
-  const int steps = pt.k / KSTEP, s0 = steps * kw / KW, s1 = steps * (kw + 1) / KW;
+  const int steps = pt.k / KSTEP, s0 = steps * wave / KW, s1 = steps * (wave + 1) / KW;
   const elem_t* wp[NR];
 #pragma unroll
   for (int r = 0; r < NR; ++r) {
@@ -84,37 +82,52 @@ __global__ __launch_bounds__(64 * NW * KW) void gemm_rows_kernel(GemmArgs p) {
     for (int r = 0; r < NR; ++r)
 #pragma unroll
       for (int m = 0; m < MB; ++m) acc[r][m] = zero4();
-    frag_t wf[NR][U], wn[NR][U];
-    auto request = [&](frag_t (&f)[NR][U], int s) {
+    // two sets of U steps of weights in turn (HBM), two sets of two steps of x in turn (L1 / L2), each requested one set ahead
+    frag_t wf[2][NR][U], xf[2][MB][2];
+    auto request_w = [&](frag_t (&f)[NR][U], int s) {
 #pragma unroll
       for (int u = 0; u < U; ++u)
 #pragma unroll
         for (int r = 0; r < NR; ++r) f[r][u] = __builtin_nontemporal_load((const frag_t*)(wp[r] + (int64_t)(s + u) * KSTEP));
     };
-    auto multiply = [&](frag_t (&f)[NR][U], int s) {
+    auto request_x = [&](frag_t (&f)[MB][2], int s) {
 #pragma unroll
       for (int m = 0; m < MB; ++m) {
         if (m < mb) {
-          frag_t xf[U];
+          f[m][0] = *(const frag_t*)(xp[m] + (int64_t)s * KSTEP);
+          f[m][1] = *(const frag_t*)(xp[m] + (int64_t)(s + 1) * KSTEP);
+        }
+      }
+    };
+    auto multiply = [&](frag_t (&f)[NR][U], int s) {
 #pragma unroll
-          for (int u = 0; u < U; ++u) xf[u] = *(const frag_t*)(xp[m] + (int64_t)(s + u) * KSTEP);
+      for (int u = 0; u < U; u += 2) {
+        if (s + u + 4 <= s1) request_x(xf[(u / 2 + 1) & 1], s + u + 2);
 #pragma unroll
-          for (int u = 0; u < U; ++u)
+        for (int m = 0; m < MB; ++m) {
+          if (m < mb) {
 #pragma unroll
-            for (int r = 0; r < NR; ++r) acc[r][m] = mma(f[r][u], xf[u], acc[r][m]);
+            for (int v = 0; v < 2; ++v)
+#pragma unroll
+              for (int r = 0; r < NR; ++r) acc[r][m] = mma(f[r][u + v], xf[(u / 2) & 1][m][v], acc[r][m]);
+          }
         }
       }
     };
     int s = s0;
-    if (s + U <= s1) request(wf, s);
-    while (s + U <= s1) {              // the next U steps are on their way while these multiply
-      if (s + 2 * U <= s1) request(wn, s + U);
-      multiply(wf, s);
-      s += U;
-      if (s + U > s1) break;
-      if (s + 2 * U <= s1) request(wf, s + U);
-      multiply(wn, s);
-      s += U;
+    if (s + U <= s1) {
+      request_w(wf[0], s);
+      request_x(xf[0], s);
+      while (true) {
+        if (s + 2 * U <= s1) request_w(wf[1], s + U);
+        multiply(wf[0], s);
+        s += U;
+        if (s + U > s1) break;
+        if (s + 2 * U <= s1) request_w(wf[0], s + U);
+        multiply(wf[1], s);
+        s += U;
+        if (s + U > s1) break;
+      }
     }
     for (; s < s1; ++s) {
       frag_t w1[NR];
@@ -123,19 +136,19 @@ __global__ __launch_bounds__(64 * NW * KW) void gemm_rows_kernel(GemmArgs p) {
 #pragma unroll
       for (int m = 0; m < MB; ++m) {
         if (m < mb) {
-          const frag_t xf = *(const frag_t*)(xp[m] + (int64_t)s * KSTEP);
+          const frag_t x1 = *(const frag_t*)(xp[m] + (int64_t)s * KSTEP);
 #pragma unroll
-          for (int r = 0; r < NR; ++r) acc[r][m] = mma(w1[r], xf, acc[r][m]);
+          for (int r = 0; r < NR; ++r) acc[r][m] = mma(w1[r], x1, acc[r][m]);
         }
       }
     }
 #pragma unroll
     for (int r = 0; r < NR; ++r)
 #pragma unroll
-      for (int m = 0; m < MB; ++m) *(f32x4*)&red[kw][16 * m + l15][16 * r + 4 * l4] = acc[r][m];
+      for (int m = 0; m < MB; ++m) *(f32x4*)&red[wave][16 * m + l15][16 * r + 4 * l4] = acc[r][m];
     __syncthreads();
     constexpr int OB = EPI == LM_EPI_GLU ? NR / 2 : NR;      // 16-channel blocks of the result
-    for (int i = gt; i < 16 * MB * OB * 4; i += 64 * KW) {
+    for (int i = tid; i < 16 * MB * OB * 4; i += 64 * KW) {
       const int m = i / (OB * 4), q = i - m * (OB * 4), blk = q >> 2, c4 = 4 * (q & 3);
       const int sb = EPI == LM_EPI_GLU ? 2 * blk : blk;
       if (m0 + m >= rows) continue;
@@ -153,97 +166,122 @@ __global__ __launch_bounds__(64 * NW * KW) void gemm_rows_kernel(GemmArgs p) {
   }
 }
 
-constexpr int TM = 128, TN = 128, TROWB = 128, TK = TROWB / (int)sizeof(elem_t);     // rows, channels, k bytes / values per stage
-typedef Tile<TROWB> KTile;
+constexpr int TM = LM_TILE_ROWS, TN = 128;                  // rows, channels of a tile
+constexpr int SROWB = 64, SK = SROWB / (int)sizeof(elem_t);  // a stage: 64 bytes of k of every row
+constexpr int STAGE = (TM + TN) * SROWB, STAGES = 3;
+static_assert(TM == 256, "the wave layout");
 
+// LDS rows of 64 bytes, four 16-byte slots and four rows to a 256-byte line: slot s of row r at s ^ (0, 2, 3, 1)[r / 4 % 4], with
+// the property Tile::swizzle has for fragment reads
+__device__ __forceinline__ int stage_swizzle(int row) {
+  const int q = (row >> 2) & 3;
+  return (((q ^ (q >> 1)) & 1) << 1) | (q >> 1);
+}
+
+// The LDS-DMA of a stage, hidden from the compiler: it would wait for every DMA in flight in front of the first LDS read.  The
+// loop counts the pieces itself (wait_pieces).  M0 is the compiler's: saved and restored.
+__device__ __forceinline__ void dma16_uncounted(const void* src, uint32_t lds_dst) {
+  uint32_t keep;
+  asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %2\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off\n\ts_mov_b32 m0, %0"
+               : "=&s"(keep)
+               : "v"(src), "s"(lds_dst)
+               : "memory");
+}
+template <int N>
+__device__ __forceinline__ void wait_pieces() {
+  asm volatile("s_waitcnt vmcnt(%0)" ::"n"(N) : "memory");
+}
+
+// 4 waves, 128 rows x 64 channels each; three stages: while one multiplies, two are on their way
 template <int EPI>
 __global__ __launch_bounds__(256, 2) void gemm_tiles_kernel(GemmArgs p, int mt_a, int mt_b) {
-  __shared__ __attribute__((aligned(16))) uint8_t wt0[TN * TROWB], wt1[TN * TROWB], xt0[TM * TROWB], xt1[TM * TROWB];
+  __shared__ __attribute__((aligned(16))) uint8_t lds[STAGES * STAGE];
+  __shared__ int y_row[TM];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l15 = lane & 15, l4 = lane >> 4;
-  // linear order: groups of 8 row tiles, all channel tiles of such a group before the next one; a contiguous range per XCD
+  // linear order: bands of row tiles, all channel tiles of a band before the next one; of both parts a contiguous range per XCD
   const int nt_a = (p.a.n + TN - 1) / TN, nt_b = mt_b ? (p.b.n + TN - 1) / TN : 0;
-  const int mt = p.tiles ? p.n_tiles[0] : mt_a;              // row tiles of part a that exist
-  int id = xcd_contiguous(blockIdx.x, mt_a * nt_a + mt_b * nt_b);
-  if (id < 0) return;
-  const bool is_b = id >= mt_a * nt_a;
+  const int wgs_b = 8 * ((mt_b * nt_b + 7) >> 3);
+  const bool is_b = (int)blockIdx.x < wgs_b;
   const Part& pt = is_b ? p.b : p.a;
   const int nt = is_b ? nt_b : nt_a, mts = is_b ? mt_b : mt_a;
-  if (is_b) id -= mt_a * nt_a;
-  constexpr int GM = 8;
+  const int id = xcd_contiguous(is_b ? blockIdx.x : blockIdx.x - wgs_b, mts * nt);
+  if (id < 0) return;
+  constexpr int GM = 4;
   const int band = id / (GM * nt), in = id - band * GM * nt, bm = min(GM, mts - band * GM);
   const int mi = band * GM + in % bm, ni = in / bm;
-  if (!is_b && mi >= mt) return;
   const int* perm = is_b ? nullptr : p.perm;
-  int first, rows, g = 0;
+  int first = mi * TM, rows, g = 0;
   if (perm) {
-    g = p.tiles[2 * mi];
-    first = p.tiles[2 * mi + 1];
-    rows = p.off[g + 1] - first;
+    const i32x4 t = *(const i32x4*)(p.tiles + 4 * mi);       // group, first place, rows
+    if (t[2] <= 0) return;
+    g = t[0];
+    first = t[1];
+    rows = t[2];
   } else {
-    first = mi * TM;
-    rows = (is_b ? p.rows_b : p.rows_a) - first;
+    rows = min(TM, (is_b ? p.rows_b : p.rows_a) - first);
   }
-  rows = min(rows, TM);
   const int n0 = ni * TN;
   const elem_t* w = pt.w + (int64_t)g * pt.n * pt.k;
-  // DMA pieces of 8 rows: lane -> (row lane / 8, physical slot lane % 8); wave w carries pieces 4 w .. 4 w + 3 of both operands
-  const elem_t *wsrc[4], *xsrc[4];
+  // pieces of 16 rows: lane -> (row lane / 4, physical slot lane % 4); a wave carries 2 of the weights' and 4 of x's
+  const elem_t *wsrc[2], *xsrc[4];
+  const int pr = lane >> 2, ps = (lane & 3) ^ stage_swizzle(pr);
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
-    const int r = 8 * (4 * wave + i) + (lane >> 3), s = (lane & 7) ^ KTile::swizzle(r);
-    const int c = n0 + r < pt.n ? n0 + r : pt.n - 1;
-    wsrc[i] = w + (int64_t)c * pt.k + s * FR;
-    const int rr = r < rows ? r : rows - 1;
-    const int xr = perm ? perm[first + rr] / p.x_div : first + rr;
-    xsrc[i] = pt.x + (int64_t)xr * pt.ldx + s * FR;
+    const int r = min(16 * (4 * wave + i) + pr, rows - 1);
+    const int xr = perm ? perm[first + r] / p.x_div : first + r;
+    xsrc[i] = pt.x + (int64_t)xr * pt.ldx + ps * FR;
   }
-  auto stage = [&](uint8_t* wt, uint8_t* xt, int k0) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      dma16(wsrc[i] + k0, wt + 1024 * (4 * wave + i));
-      dma16(xsrc[i] + k0, xt + 1024 * (4 * wave + i));
-    }
+  for (int i = 0; i < 2; ++i) wsrc[i] = w + (int64_t)min(n0 + 16 * (2 * wave + i) + pr, pt.n - 1) * pt.k + ps * FR;
+  y_row[tid] = tid < rows ? (perm ? perm[first + tid] : first + tid) : -1;
+  const uint32_t lds0 = (uint32_t)(size_t)(__attribute__((address_space(3))) uint8_t*)lds;
+  const int uw = __builtin_amdgcn_readfirstlane(wave);
+  auto stage = [&](int st, int k0) {
+    const uint32_t dst = lds0 + st * STAGE;
+#pragma unroll
+    for (int i = 0; i < 2; ++i) dma16_uncounted(wsrc[i] + k0, dst + 1024 * (2 * uw + i));
+#pragma unroll
+    for (int i = 0; i < 4; ++i) dma16_uncounted(xsrc[i] + k0, dst + TN * SROWB + 1024 * (4 * uw + i));
   };
-  const int wn = 64 * (wave & 1), wm = 64 * (wave >> 1);
-  f32x4 acc[4][4];
+  const int wn = 64 * (wave & 1), wm = 128 * (wave >> 1);
+  f32x4 acc[4][8];
 #pragma unroll
   for (int i = 0; i < 4; ++i)
 #pragma unroll
-    for (int j = 0; j < 4; ++j) acc[i][j] = zero4();
-  stage(wt0, xt0, 0);
-  __syncthreads();
-  auto step = [&](const uint8_t* wt, const uint8_t* xt, uint8_t* wnext, uint8_t* xnext, int knext) {
-    frag_t a[2][4], b[2][4];
+    for (int j = 0; j < 8; ++j) acc[i][j] = zero4();
+  const int nk = pt.k / SK;                                 // (>= 2: k is a multiple of 64)
+  const int lane_off = l15 * SROWB + ((l4 ^ stage_swizzle(l15)) << 4);
+  wait_pieces<0>();                                         // the compiler's own loads
+  stage(0, 0);
+  stage(1, SK);
+  int st = 0;
+  for (int t = 0; t < nk; ++t) {
+    if (t + 1 < nk) wait_pieces<6>();                       // stage t is there, the 6 pieces of t + 1 may still fly
+    else wait_pieces<0>();
+    __builtin_amdgcn_s_barrier();                           // ... for every wave, and everyone has left stage t - 1
+    asm volatile("" ::: "memory");
+    if (t + 2 < nk) stage(st == 0 ? 2 : st - 1, (t + 2) * SK);
+    const uint8_t* wt = lds + st * STAGE + wn * SROWB + lane_off;
+    const uint8_t* xt = lds + st * STAGE + (TN + wm) * SROWB + lane_off;
+    frag_t a[4], b[8];
 #pragma unroll
-    for (int s = 0; s < 2; ++s)
+    for (int i = 0; i < 4; ++i) a[i] = *(const frag_t*)(wt + 16 * SROWB * i);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        a[s][i] = KTile::frag(wt, wn + 16 * i + l15, 4 * s + l4);
-        b[s][i] = KTile::frag(xt, wm + 16 * i + l15, 4 * s + l4);
-      }
-    __builtin_amdgcn_sched_barrier(0);
-    if (knext < pt.k) stage(wnext, xnext, knext);
-    __builtin_amdgcn_sched_barrier(0);
+    for (int j = 0; j < 8; ++j) b[j] = *(const frag_t*)(xt + 16 * SROWB * j);
     __builtin_amdgcn_s_setprio(1);
 #pragma unroll
-    for (int s = 0; s < 2; ++s)
+    for (int j = 0; j < 8; ++j)
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
-#pragma unroll
-        for (int j = 0; j < 4; ++j) acc[i][j] = mma(a[s][i], b[s][j], acc[i][j]);
+      for (int i = 0; i < 4; ++i) acc[i][j] = mma(a[i], b[j], acc[i][j]);
     __builtin_amdgcn_s_setprio(0);
-    __syncthreads();
-  };
-  for (int k0 = 0; k0 < pt.k; k0 += 2 * TK) {
-    step(wt0, xt0, wt1, xt1, k0 + TK);
-    if (k0 + TK < pt.k) step(wt1, xt1, wt0, xt0, k0 + 2 * TK);
+    st = st == 2 ? 0 : st + 1;
   }
+  __syncthreads();                                          // the stages are free
   if constexpr (EPI == LM_EPI_F32) {
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const int m = wm + 16 * j + l15;
-      if (m >= rows) continue;
-      const int64_t row = perm ? perm[first + m] : first + m;
+    for (int j = 0; j < 8; ++j) {
+      const int row = y_row[wm + 16 * j + l15];
+      if (row < 0) continue;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int c = n0 + wn + 16 * i + 4 * l4;
@@ -251,16 +289,15 @@ __global__ __launch_bounds__(256, 2) void gemm_tiles_kernel(GemmArgs p, int mt_a
       }
     }
   } else {
-    // through LDS, so that a row leaves in whole 16-byte pieces of neighbouring lanes; a wave handles its own 64 rows x (64 or
-    // 32) channels in two halves of 32 rows (all tiles have been read: the last step ended with a barrier)
+    // through LDS, so that a row leaves in whole 16-byte pieces of neighbouring lanes: 32 rows of the wave's at a time
     constexpr int OC = EPI == LM_EPI_GLU ? 32 : 64, PITCH = OC * (int)sizeof(elem_t) + 16, PPR = OC / FR;
-    uint8_t* buf = wave == 0 ? wt0 : wave == 1 ? wt1 : wave == 2 ? xt0 : xt1;
-    static_assert(32 * PITCH <= TN * TROWB, "a wave's half fits its buffer");
+    static_assert(4 * 32 * PITCH <= STAGES * STAGE, "the waves' buffers");
+    uint8_t* buf = lds + wave * 32 * PITCH;
 #pragma unroll
-    for (int half = 0; half < 2; ++half) {
+    for (int part = 0; part < 4; ++part) {
 #pragma unroll
       for (int jj = 0; jj < 2; ++jj) {
-        const int j = 2 * half + jj;
+        const int j = 2 * part + jj;
 #pragma unroll
         for (int i = 0; i < 4; i += EPI == LM_EPI_GLU ? 2 : 1) {
           f32x4 v = acc[i][j];
@@ -278,11 +315,9 @@ __global__ __launch_bounds__(256, 2) void gemm_tiles_kernel(GemmArgs p, int mt_a
 #pragma unroll
       for (int i = 0; i < 32 * PPR / 64; ++i) {
         const int pc = 64 * i + lane, r = pc / PPR, q = pc % PPR;
-        const int m = wm + 32 * half + r, c = (EPI == LM_EPI_GLU ? (n0 + wn) / 2 : n0 + wn) + q * FR;
-        if (m < rows && c < (EPI == LM_EPI_GLU ? pt.n / 2 : pt.n)) {
-          const int64_t row = perm ? perm[first + m] : first + m;
-          *(frag_t*)((elem_t*)pt.y + row * pt.ldy + c) = *(const frag_t*)(buf + r * PITCH + q * 16);
-        }
+        const int row = y_row[wm + 32 * part + r], c = (EPI == LM_EPI_GLU ? (n0 + wn) / 2 : n0 + wn) + q * FR;
+        if (row >= 0 && c < (EPI == LM_EPI_GLU ? pt.n / 2 : pt.n))
+          *(frag_t*)((elem_t*)pt.y + (int64_t)row * pt.ldy + c) = *(const frag_t*)(buf + r * PITCH + q * 16);
       }
       __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
       __builtin_amdgcn_wave_barrier();
@@ -306,35 +341,34 @@ static int fill(GemmArgs& a, const LmGemmPart* pa, const LmGemmPart* pb, int gro
   a.b = pb ? conv(pb) : Part{};
   if (check_part(a.a, epi) || (pb && check_part(a.b, epi))) return LM_EINVAL;
   a.groups = groups; a.perm = perm; a.off = off; a.rows_a = rows_a; a.rows_b = pb ? rows_b : 0; a.x_div = perm ? x_div : 1;
-  a.tiles = nullptr; a.n_tiles = nullptr; a.scale = scale;
+  a.tiles = nullptr; a.scale = scale;
   return LM_OK;
 }
 
-template <int NR, int NW, int KW, int EPI>
+template <int NR, int KW, int EPI>
 static int launch_rows(const GemmArgs& a, int max_rows, int has_b, hipStream_t s) {
   const int n = has_b && a.b.n > a.a.n ? a.b.n : a.a.n;
-  const int mb = max_rows <= 16 ? 1 : max_rows <= 32 ? 2 : 4;
-  const dim3 grid((n + 16 * NR * NW - 1) / (16 * NR * NW), a.groups + has_b, a.perm ? 1 : (max_rows + 16 * mb - 1) / (16 * mb));
-  const dim3 block(64 * NW * KW);
-  if (mb == 1) hipLaunchKernelGGL((gemm_rows_kernel<NR, 1, NW, KW, EPI>), grid, block, 0, s, a);
-  else if (mb == 2) hipLaunchKernelGGL((gemm_rows_kernel<NR, 2, NW, KW, EPI>), grid, block, 0, s, a);
-  else hipLaunchKernelGGL((gemm_rows_kernel<NR, 4, NW, KW, EPI>), grid, block, 0, s, a);
+  const int mb = max_rows <= 16 || (n <= 256 && !a.perm && max_rows <= 64) ? 1 : max_rows <= 32 ? 2 : 4;
+  const dim3 grid((n + 16 * NR - 1) / (16 * NR), a.groups + has_b, a.perm ? 1 : (max_rows + 16 * mb - 1) / (16 * mb));
+  const dim3 block(64 * KW);
+  if (mb == 1) hipLaunchKernelGGL((gemm_rows_kernel<NR, 1, KW, EPI>), grid, block, 0, s, a);
+  else if (mb == 2) hipLaunchKernelGGL((gemm_rows_kernel<NR, 2, KW, EPI>), grid, block, 0, s, a);
+  else hipLaunchKernelGGL((gemm_rows_kernel<NR, 4, KW, EPI>), grid, block, 0, s, a);
   return launch_status();
 }
 
-// Channels per workgroup: as many as still leave a workgroup for every CU (fewer reads of x).  A product of few channels over
-// many rows (the router of a prompt) has its workgroups along the rows instead.
+// Channels per workgroup: the more the fewer reads of x, as long as every CU has work.  A product of few channels over many rows
+// (the router of a prompt) has its workgroups along the rows instead.
 template <int EPI>
 static int plan_rows(const GemmArgs& a, int max_rows, int has_b, hipStream_t s) {
   const int64_t n = (int64_t)a.groups * a.a.n;
   if constexpr (EPI == LM_EPI_GLU) {
-    return launch_rows<2, 1, 8, EPI>(a, max_rows, has_b, s);
+    return n >= 64 * 256 ? launch_rows<4, 4, EPI>(a, max_rows, has_b, s) : launch_rows<2, 8, EPI>(a, max_rows, has_b, s);
   } else {
-    if (max_rows > 64) return launch_rows<2, 1, 8, EPI>(a, max_rows, has_b, s);
-    if (n >= 128 * 256) return launch_rows<2, 4, 2, EPI>(a, max_rows, has_b, s);
-    if (n >= 64 * 240) return launch_rows<1, 4, 2, EPI>(a, max_rows, has_b, s);
-    if (n >= 32 * 240) return launch_rows<1, 2, 4, EPI>(a, max_rows, has_b, s);
-    return launch_rows<1, 1, 8, EPI>(a, max_rows, has_b, s);
+    if (max_rows > 64) return launch_rows<2, 8, EPI>(a, max_rows, has_b, s);
+    if (n >= 64 * 512 || (n >= 64 * 150 && max_rows > 16)) return launch_rows<4, 4, EPI>(a, max_rows, has_b, s);
+    if (n >= 64 * 150) return launch_rows<2, 4, EPI>(a, max_rows, has_b, s);
+    return launch_rows<1, 8, EPI>(a, max_rows, has_b, s);
   }
 }
 
@@ -353,17 +387,16 @@ extern "C" int lm_gemm_rows(const LmGemmPart* pa, const LmGemmPart* pb, int grou
 }
 
 extern "C" int lm_gemm_tiles(const LmGemmPart* pa, const LmGemmPart* pb, int groups, const int* perm, const int* off,
-                             const int* tiles, const int* n_tiles, int max_tiles, int rows_a, int rows_b, int x_div,
+                             const int* tiles, int max_tiles, int rows_a, int rows_b, int x_div,
                              float scale, int epi, void* stream) {
   GemmArgs a;
   if (fill(a, pa, pb, groups, perm, off, rows_a, rows_b, x_div, scale, epi)) return LM_EINVAL;
-  if (perm && (!tiles || !n_tiles || max_tiles <= 0)) return LM_EINVAL;
+  if (perm && (!tiles || max_tiles <= 0)) return LM_EINVAL;
   a.tiles = perm ? tiles : nullptr;
-  a.n_tiles = n_tiles;
   const int mt_a = perm ? max_tiles : (rows_a + TM - 1) / TM, mt_b = pb && rows_b > 0 ? (rows_b + TM - 1) / TM : 0;
-  const int64_t total = (int64_t)mt_a * ((a.a.n + TN - 1) / TN) + (int64_t)mt_b * (mt_b ? (a.b.n + TN - 1) / TN : 0);
-  if (total <= 0 || total > (1 << 30)) return LM_EINVAL;
-  const dim3 grid((unsigned)(8 * ((total + 7) / 8)));
+  const int64_t tiles_a = (int64_t)mt_a * ((a.a.n + TN - 1) / TN), tiles_b = mt_b ? (int64_t)mt_b * ((a.b.n + TN - 1) / TN) : 0;
+  if (tiles_a <= 0 || tiles_a + tiles_b > (1 << 30)) return LM_EINVAL;
+  const dim3 grid((unsigned)(8 * ((tiles_a + 7) / 8) + 8 * ((tiles_b + 7) / 8)));
   hipStream_t s = (hipStream_t)stream;
   if (epi == LM_EPI_ELEM) hipLaunchKernelGGL((gemm_tiles_kernel<LM_EPI_ELEM>), grid, dim3(256), 0, s, a, mt_a, mt_b);
   else if (epi == LM_EPI_F32) hipLaunchKernelGGL((gemm_tiles_kernel<LM_EPI_F32>), grid, dim3(256), 0, s, a, mt_a, mt_b);

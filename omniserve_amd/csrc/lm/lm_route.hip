@@ -1,5 +1,5 @@
 // Expert choice and the order of the grouped products: per token the `top` largest router logits (ties: the lower expert) and
-// their softmax; then the (token, choice) pairs sorted by expert -- off[experts + 1], perm[pairs] -- and the 128-row tiles of
+// their softmax; then the (token, choice) pairs sorted by expert -- off[experts + 1], perm[pairs] -- and the row tiles of
 // every expert for lm_gemm_tiles.
 #include "lm_common.h"
 #include "omniserve_lm.h"
@@ -9,39 +9,48 @@ namespace lm {
 constexpr int MAX_EXPERTS = 512, MAX_TOP = 16;
 constexpr int CHOOSE_TOKENS = 16;      // tokens per workgroup of route_choose_kernel
 
-// one wave per token; lane l looks at its EPL experts l, l + 64, ...; every lane ends up with the same choices
+// one wave per token; lane l holds its EPL experts l, l + 64, ... and counts for each how many come before it in the order
+// (larger logit, then lower number): the first `top` are the choice
 template <int EPL>
 __device__ __forceinline__ void choose(const float* z, const float* bias, int experts, int top, int lane, int* ids, float* wts) {
   float v[EPL];
+  int before[EPL];
 #pragma unroll
   for (int i = 0; i < EPL; ++i) {
     const int e = lane + 64 * i;
-    v[i] = e < experts ? z[e] + (bias ? bias[e] : 0.f) : -INFINITY;
+    const float x = e < experts ? z[e] + (bias ? bias[e] : 0.f) : -INFINITY;
+    v[i] = x == x ? x : -INFINITY;        // (NaN: last)
+    before[i] = 0;
   }
-  float best0 = 0.f, sum = 0.f, mine = 0.f;
-  int my_id = 0;
-  for (int k = 0; k < top; ++k) {
-    float b = -INFINITY;
-    int at = 0x7fffffff;
 #pragma unroll
-    for (int i = 0; i < EPL; ++i)
-      if (v[i] > b) { b = v[i]; at = lane + 64 * i; }
+  for (int b = 0; b < EPL; ++b) {
+    const int n = min(64, experts - 64 * b);
+    for (int l = 0; l < n; ++l) {
+      const float o = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v[b]), l));
+      const int oe = 64 * b + l;
 #pragma unroll
-    for (int m = 32; m > 0; m >>= 1) {
-      const float ob = __shfl_xor(b, m, 64);
-      const int oa = __shfl_xor(at, m, 64);
-      if (ob > b || (ob == b && oa < at)) { b = ob; at = oa; }
+      for (int i = 0; i < EPL; ++i) before[i] += (int)(o > v[i]) | ((int)(o == v[i]) & (int)(oe < lane + 64 * i));
     }
-    if (at >= experts) at = k;        // only NaN logits get here: any in-range expert
-    if (k == 0) best0 = b;
-    const float ex = __expf(b - best0);
-    sum += ex;
-    if (lane == k) { mine = ex; my_id = at; }
-#pragma unroll
-    for (int i = 0; i < EPL; ++i)
-      if (at == lane + 64 * i) v[i] = -INFINITY;
   }
-  if (lane < top) { ids[lane] = my_id; wts[lane] = mine / sum; }
+  float best = v[0];
+#pragma unroll
+  for (int i = 1; i < EPL; ++i) best = fmaxf(best, v[i]);
+#pragma unroll
+  for (int m = 32; m > 0; m >>= 1) best = fmaxf(best, __shfl_xor(best, m, 64));
+  if (best == -INFINITY) best = 0.f;
+  float ex[EPL], sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < EPL; ++i) {
+    ex[i] = before[i] < top ? __expf(v[i] - best) : 0.f;
+    sum += ex[i];
+  }
+  sum = wave_sum(sum);
+#pragma unroll
+  for (int i = 0; i < EPL; ++i)
+    if (before[i] < top && lane + 64 * i < experts) {
+      ids[before[i]] = lane + 64 * i;
+      wts[before[i]] = ex[i] / sum;
+    }
 }
 
 // everything for up to 64 tokens in one workgroup
@@ -106,10 +115,10 @@ __global__ __launch_bounds__(256) void route_choose_kernel(const float* z, int64
   }
 }
 
-// ... offsets and row tiles ...
-__global__ __launch_bounds__(512) void route_offsets_kernel(const int* count, int experts, int* off, int* tiles, int* n_tiles) {
+// ... offsets and row tiles (entries past the last tile: no rows) ...
+__global__ __launch_bounds__(512) void route_offsets_kernel(const int* count, int experts, int max_tiles, int* off, int* tiles) {
   __shared__ int s_off[MAX_EXPERTS], s_tile[MAX_EXPERTS];
-  const int e = threadIdx.x, c = e < experts ? count[e] : 0, nt = (c + 127) / 128;
+  const int e = threadIdx.x, c = e < experts ? count[e] : 0, nt = (c + LM_TILE_ROWS - 1) / LM_TILE_ROWS;
   s_off[e] = c;
   s_tile[e] = nt;
   __syncthreads();
@@ -120,18 +129,14 @@ __global__ __launch_bounds__(512) void route_offsets_kernel(const int* count, in
     s_tile[e] += b;
     __syncthreads();
   }
+  i32x4* out = (i32x4*)tiles;
   if (e < experts) {
     const int o = s_off[e] - c, t = s_tile[e] - nt;
     off[e] = o;
-    for (int i = 0; i < nt; ++i) {
-      tiles[2 * (t + i)] = e;
-      tiles[2 * (t + i) + 1] = o + 128 * i;
-    }
-    if (e == experts - 1) {
-      off[experts] = s_off[e];
-      n_tiles[0] = s_tile[e];
-    }
+    for (int i = 0; i < nt; ++i) out[t + i] = (i32x4){e, o + LM_TILE_ROWS * i, min(LM_TILE_ROWS, c - LM_TILE_ROWS * i), 0};
+    if (e == experts - 1) off[experts] = s_off[e];
   }
+  for (int t = s_tile[511] + e; t < max_tiles; t += 512) out[t] = (i32x4){0, 0, 0, 0};
 }
 
 // ... and the pairs in their places
@@ -152,11 +157,11 @@ using namespace lm;
 extern "C" int64_t lm_route_scratch_words(int tokens, int experts, int top) { return MAX_EXPERTS + 2 * (int64_t)tokens * top; }
 extern "C" int lm_route_max_tiles(int tokens, int experts, int top) {
   const int64_t pairs = (int64_t)tokens * top;
-  return (int)(pairs / 128 + (pairs < experts ? pairs : experts));
+  return (int)(pairs / LM_TILE_ROWS + (pairs < experts ? pairs : experts));
 }
 
 extern "C" int lm_route(const float* z, int64_t ldz, const float* bias, int tokens, int experts, int top, float* wts, int* off,
-                        int* perm, int* tiles, int* n_tiles, int* scratch_i32, void* stream) {
+                        int* perm, int* tiles, int* scratch_i32, void* stream) {
   if (tokens <= 0 || experts <= 0 || experts > MAX_EXPERTS || top <= 0 || top > MAX_TOP || top > experts || ldz < experts ||
       (int64_t)tokens * top > (1 << 28))
     return LM_EINVAL;
@@ -166,13 +171,14 @@ extern "C" int lm_route(const float* z, int64_t ldz, const float* bias, int toke
     hipLaunchKernelGGL(k, dim3(1), dim3(1024), 0, s, z, ldz, bias, tokens, experts, top, wts, off, perm);
     return launch_status();
   }
-  if (!tiles || !n_tiles || !scratch_i32) return LM_EINVAL;
+  if (!tiles || !scratch_i32) return LM_EINVAL;
   const int pairs = tokens * top;
   int *count = scratch_i32, *ids = count + MAX_EXPERTS, *rank = ids + pairs;
   hipLaunchKernelGGL(clear_kernel, dim3(1), dim3(512), 0, s, count, MAX_EXPERTS);
   auto k = experts <= 64 ? route_choose_kernel<1> : experts <= 128 ? route_choose_kernel<2> : route_choose_kernel<MAX_EXPERTS / 64>;
   hipLaunchKernelGGL(k, dim3((tokens + CHOOSE_TOKENS - 1) / CHOOSE_TOKENS), dim3(256), 0, s, z, ldz, bias, tokens, experts, top, wts, ids, rank, count);
-  hipLaunchKernelGGL(route_offsets_kernel, dim3(1), dim3(512), 0, s, count, experts, off, tiles, n_tiles);
+  hipLaunchKernelGGL(route_offsets_kernel, dim3(1), dim3(512), 0, s, count, experts,
+                     lm_route_max_tiles(tokens, experts, top), off, tiles);
   hipLaunchKernelGGL(route_scatter_kernel, dim3((pairs + 255) / 256), dim3(256), 0, s, ids, rank, off, pairs, perm);
   return launch_status();
 }

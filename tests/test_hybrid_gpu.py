@@ -195,7 +195,7 @@ def test_far_key_of_the_recurrent_state(dtype):
 # feed-forward, norms, products, routing
 # ---------------------------------------------------------------------------------------------------------------
 @pytest.mark.parametrize("dtype", DTYPES, ids=str)
-@pytest.mark.parametrize("tokens", [1, 7, 16, 33, 64, 65, 300])
+@pytest.mark.parametrize("tokens", [1, 7, 16, 33, 64, 65, 300, 1200])
 @pytest.mark.parametrize("kind", [dict(), dict(top=1, shared=None), dict(experts=5, top=5, ff=130, shared=16), dict(experts=70, top=8)], ids=str)
 def test_mixture(kind, tokens, dtype):
     from omniserve_amd.backend.lm import lm_ops
@@ -243,7 +243,7 @@ def test_residual_norm(kind, width, dtype):
 
 @pytest.mark.parametrize("dtype", DTYPES, ids=str)
 @pytest.mark.parametrize("m,n,k", [(1, 304, 64), (16, 1024, 192), (17, 48, 1024), (50, 25600, 128), (64, 80, 4096), (130, 144, 192),
-                                   (700, 528, 320)])
+                                   (700, 528, 320), (257, 16, 64), (1000, 32, 1024)])
 def test_products(m, n, k, dtype):
     from omniserve_amd.backend.lm import lm_ops
     ops = lm_ops(dtype)
@@ -257,13 +257,13 @@ def test_products(m, n, k, dtype):
 def test_routing_ties_and_order():
     from omniserve_amd.backend.lm import lm_ops
     ops = lm_ops(F32)
-    for T in (3, 64, 65, 1000):
+    for T in (3, 64, 65, 1000, 5000):
         g = np.random.default_rng(17)
         z = g.integers(0, 4, (T, 40)).astype(np.float32)           # many ties
         bias = g.integers(0, 2, 40).astype(np.float32)
         zt = torch.zeros((T, 48), device=DEV)
         zt[:, :40] = torch.from_numpy(z)
-        wts, (off, perm, tiles, n_tiles, _, top) = ops.route(zt, torch.from_numpy(bias).to(DEV), 40, 3)
+        wts, (off, perm, tiles, _, top) = ops.route(zt, torch.from_numpy(bias).to(DEV), 40, 3)
         ids, wt = hybrid.route(np.eye(40)[np.zeros(T, int)] * 0 + z, np.eye(40), bias, 3)
         off, perm = off.cpu().numpy(), perm.cpu().numpy()
         assert np.abs(wts.cpu().numpy() - wt).max() < 1e-6
@@ -272,8 +272,8 @@ def test_routing_ties_and_order():
         for e in range(40):
             assert sorted(perm[off[e]:off[e + 1]]) == np.nonzero(flat == e)[0].tolist()
         if tiles is not None:
-            t = tiles.cpu().numpy()[:int(n_tiles[0])].tolist()
-            assert t == [[e, p] for e in range(40) for p in range(off[e], off[e + 1], 128)]
+            t = [r for r in tiles.cpu().numpy().tolist() if r[2]]
+            assert t == [[e, p, min(256, off[e + 1] - p), 0] for e in range(40) for p in range(off[e], off[e + 1], 256)]
 
 
 # ---------------------------------------------------------------------------------------------------------------
