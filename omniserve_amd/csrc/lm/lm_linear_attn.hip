@@ -33,7 +33,7 @@ struct LinGeom {
   static constexpr int NQ = C * KB / (16 * TH), NV = C * VB / (16 * TH);         // 16-byte loads per thread
 };
 
-constexpr int linear_waves_per_simd(int dk) { return SPLIT && dk <= 128 ? 2 : 1; }      // what the registers allow
+constexpr int linear_waves_per_simd(int dk, int waves) { return SPLIT && (dk <= 64 || waves == 8) ? 2 : 1; }      // what the registers allow
 
 __device__ __forceinline__ frag_t activate(frag_t v, int act) {
   if (act == LM_ACT_SILU) {
@@ -44,7 +44,7 @@ __device__ __forceinline__ frag_t activate(frag_t v, int act) {
 }
 
 template <int DK, int NWV, bool OUTPUT>
-__global__ __launch_bounds__(64 * NWV, linear_waves_per_simd(DK)) void linear_prefill_kernel(LinArgs p) {
+__global__ __launch_bounds__(64 * NWV, linear_waves_per_simd(DK, NWV)) void linear_prefill_kernel(LinArgs p) {
   typedef LinGeom<DK, NWV> Gm;
   typedef Tile<Gm::KB> KT;
   typedef Tile<Gm::VB> VT;

@@ -40,10 +40,7 @@ class Cache:
         self.paged = bool(model.kv_shapes())
         if not self.paged:
             num_pages = 0
-        # zeros: places of a page past its sequence's end are multiplied with a probability of zero and must be finite
-        self.kv = [(torch.zeros((num_pages, g, self.page_size, dk), dtype=model.dtype, device=device),
-                    torch.zeros((num_pages, g, self.page_size, dv), dtype=model.dtype, device=device))
-                   for g, dk, dv in model.kv_shapes()]
+        self.kv = model.page_pools(num_pages, device)
         self.state = [torch.zeros((num_slots, h, dk, dv), dtype=torch.float32, device=device) for h, dk, dv in model.state_shapes()]
         self._pages: List[int] = list(range(num_pages))[::-1]
         self._slots: List[int] = list(range(num_slots))[::-1]

@@ -44,9 +44,9 @@ class Engine:
         self.model, self.device = model, torch.device(model.device)
         self.cache = Cache(model, -(-max_tokens // model.page_size), max_seqs, self.device)
         self.builder = BatchBuilder(model, self.device)
-        self.scheduler = Scheduler(self.cache, max_batch_tokens, model.whole_prompts_only)
+        self.scheduler = Scheduler(self.cache, max_batch_tokens)
         self.sampler = Sampler(model, self.device)
-        self.use_graphs = use_graphs
+        self.use_graphs = use_graphs and model.capturable
         self._graphs: Dict[tuple, tuple] = {}
         self._next_id = 0
 

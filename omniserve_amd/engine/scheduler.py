@@ -30,8 +30,8 @@ class Request:
 
 
 class Scheduler:
-    def __init__(self, cache: Cache, max_batch_tokens: int, whole_prompts_only: bool = False):
-        self.cache, self.max_batch_tokens, self.whole_prompts_only = cache, max_batch_tokens, whole_prompts_only
+    def __init__(self, cache: Cache, max_batch_tokens: int):
+        self.cache, self.max_batch_tokens = cache, max_batch_tokens
         self.waiting: Deque[Request] = deque()
         self.running: List[Request] = []           # oldest first
 
@@ -103,8 +103,6 @@ class Scheduler:
             r = self.waiting[0]
             seq = self.cache.open()
             n = self._fitting(seq, min(len(r.tokens), budget))
-            if self.whole_prompts_only and n < len(r.tokens) and plan:
-                n = 0
             if n == 0:
                 self.cache.close(seq)
                 break

@@ -9,6 +9,7 @@ import os
 # architecture name -> (module, class)
 _REGISTRY = {
     "Bobavik": ("omniserve_amd.models.bobavik", "Bobavik"),
+    "LlamaForCausalLM": ("omniserve_amd.models.qserve_llama", "QServeLlama"),
 }
 
 

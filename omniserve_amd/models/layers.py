@@ -14,6 +14,7 @@ import torch
 
 from ..backend.lm import ATTN_ROWS, PAGE, LmOps
 from ..rope import inverse_frequencies
+from .base import EngineModel
 
 NO_WINDOW = 1 << 30
 
@@ -62,8 +63,8 @@ class LinearAttentionSpec:
     def __post_init__(self):
         if len(self.decay) != self.heads:
             raise ValueError("one decay per head")
-        if not all(0.0 < d <= 1.0 for d in self.decay):
-            raise ValueError("decays lie in (0, 1]")
+        if not all(0.0 <= d <= 1.0 for d in self.decay):
+            raise ValueError("decays lie in [0, 1]")
 
 
 @dataclasses.dataclass(frozen=True)
@@ -245,7 +246,7 @@ class LinearAttention:
         self.g0 = 2 * H * self.dk + H * self.dv
         self.w_out = pad_in_heads(w.matrix("o", width, H * s.vdim), H, s.vdim, W)
         self.norm = pad_in_heads(w.vector("norm", H * s.vdim)[None], H, s.vdim, 1)[0].contiguous()
-        self.log2_decay = torch.tensor([math.log2(d) for d in s.decay], dtype=torch.float64).to(device=w.device, dtype=torch.float32)
+        self.log2_decay = torch.tensor([math.log2(d) if d > 0 else -1e30 for d in s.decay], dtype=torch.float64).to(device=w.device, dtype=torch.float32)
 
     def state_shape(self):
         return self.s.heads, self.dk, self.dv
@@ -311,14 +312,13 @@ class Layer:
                                                                    ("norm1", "norm1b"))}
 
 
-class Decoder:
+class Decoder(EngineModel):
     """A stack of layers with a norm before and after every sublayer over an f32 residual stream.
 
     One fused launch per sublayer boundary: norm of the sublayer's output, addition, norm for the next sublayer."""
 
     page_size, attn_rows = PAGE, ATTN_ROWS
     dtypes = (torch.bfloat16, torch.float32)
-    whole_prompts_only = False
 
     def __init__(self, spec: DecoderSpec, w: Weights, ops: LmOps):
         self.spec, self.ops, self.device, self.dtype, self.vocab = spec, ops, w.device, w.dtype, spec.vocab
@@ -345,18 +345,14 @@ class Decoder:
         return [l.mixer.state_shape() for l in self.layers if not l.is_attention]
 
     def window(self):
-        """Tokens before the newest one that some layer may still read, plus one; None: all of them."""
         ws = [l.mixer.s.window for l in self.layers if l.is_attention]
         return None if any(x is None for x in ws) else max(ws, default=1)
 
     def linear_workgroups(self):
-        """Fewest workgroups one segment of a prompt gives to a recurrent layer."""
         return min((h * dv // 64 for h, _, dv in self.state_shapes()), default=0)
 
     # ---- one step ----
     def forward(self, b, cache):
-        """b: engine.batch.DeviceBatch.  Runs the step's tokens from the cache and state of earlier steps; returns the logits
-        f32 [wanted rows, vocab] (None when no row is wanted)."""
         ops, spec, W = self.ops, self.spec, self.W
         T = b.tokens.numel()
         x = torch.empty((T, W), dtype=torch.float32, device=self.device)

@@ -14,6 +14,7 @@ from omniserve_amd.engine import Engine, SamplingParams, SequenceInput
 from omniserve_amd.engine.cache import Cache, OutOfPages
 from omniserve_amd.engine.sampling import filtered_probabilities
 from omniserve_amd.models import bobavik, layers
+from omniserve_amd.models.base import EngineModel
 from omniserve_amd.rope import inverse_frequencies
 from oracle import hybrid
 from tests.hybrid_util import attention, config, lightning, moe, random_state, tensors
@@ -21,9 +22,9 @@ from tests.hybrid_util import attention, config, lightning, moe, random_state, t
 CPU = torch.device("cpu")
 
 
-class Pages:
+class Pages(EngineModel):
     """Next token = hash of the last `span` tokens (read back through the block table) and of the state's sum of all tokens."""
-    page_size, attn_rows, vocab, dtype, device, whole_prompts_only = 64, 128, 97, torch.float32, CPU, False
+    vocab, dtype, device = 97, torch.float32, CPU
 
     def __init__(self, span=None):
         self.span = span
@@ -189,7 +190,7 @@ def test_registry_and_config():
     assert (a.window, a.rotary.dims, a.rotary.base, a.value_mix, a.rotary.scaling["factor"]) == (9, 16, 777.0, True, 8.0)
     assert b.decay == (0.55, 0.93, 0.9985) and spec.layers[1].moe is None
     assert not c.value_mix and c.rotary.scaling is None and spec.layers[2].moe == layers.MoeSpec(6, 1, 48, None)
-    for bad in (dict(attention(), type="other"), dict(attention(), mlp={"kind": "dense"}), lightning(decay=[0.5, 1.5, 0.1]),
+    for bad in (dict(attention(), type="other"), dict(attention(), mlp={"kind": "dense"}), lightning(decay=[0.5, 1.5, 0.1]), lightning(decay=[0.5, 0.2]),
                 attention(heads=3, kv_heads=2), attention(scale=-1.0), attention(window=0), attention(rot=50)):
         with pytest.raises(ValueError):
             bobavik.parse_config(config([bad]))
@@ -274,3 +275,24 @@ def test_trace_replay_rejects_what_it_cannot_run(tmp_path):
     r = subprocess.run([sys.executable, os.path.join(root, "bin", "trace_run"), "--model", str(tmp_path), "--dtype", "float32", "--out",
                         str(tmp_path), "--max-tokens", "64"], input="", text=True, capture_output=True, timeout=100)
     assert r.returncode not in (0, 3) and "unknown architecture" in r.stderr
+
+
+def test_command_line(tmp_path, capsys):
+    from omniserve_amd import cli
+    assert cli.main(["models"]) == 0
+    assert {"Bobavik", "LlamaForCausalLM"} <= set(capsys.readouterr().out.split())
+    a = cli.parser().parse_args(["generate", "--model", "m", "--prompt-ids", "1, 2,3", "--prompt-ids", "4", "--stop-ids", "7,8"])
+    assert a.prompt_ids == [[1, 2, 3], [4]] and a.stop_ids == [7, 8] and a.temperature == 0
+    assert cli.main(["generate", "--model", str(tmp_path)]) == 2
+    with pytest.raises(SystemExit):
+        cli.main(["generate", "--model", "m", "--prompt-ids", "x"])
+    with pytest.raises(SystemExit):
+        cli.main(["trace", "--nothing"])
+
+
+def test_llama_config():
+    from omniserve_amd.models import qserve_llama
+    c = qserve_llama.parse_config({"hidden_size": 512, "intermediate_size": 1024, "num_attention_heads": 4, "num_key_value_heads": 2,
+                                   "num_hidden_layers": 3, "vocab_size": 99, "rope_theta": 5e5, "quantization": {"group_size": 128}})
+    assert (c.head_dim, c.kv_heads, c.layers, c.group_size, c.rope_theta) == (128, 2, 3, 128, 5e5)
+    assert models.model_class({"architectures": ["LlamaForCausalLM"]}) is qserve_llama.QServeLlama

@@ -4,6 +4,7 @@ import numpy as np
 import pytest
 import torch
 
+from omniserve_amd.models.base import EngineModel
 from oracle import hybrid
 from tests.hybrid_util import (attention, config, cuts, errors, lightning, moe, random_state, random_tokens, run_alone, to_numpy)
 
@@ -17,9 +18,9 @@ DEV = torch.device("cuda:0")
 # ---------------------------------------------------------------------------------------------------------------
 # one mixer alone: h in, output out, through the cache
 # ---------------------------------------------------------------------------------------------------------------
-class OneMixer:
+class OneMixer(EngineModel):
     """A mixer with what the cache and the batch builder ask a model for."""
-    page_size, attn_rows, vocab = 64, 128, 1
+    vocab = 1
 
     def __init__(self, layer, width, dtype, seed, weights=None, mixes=False):
         from omniserve_amd.backend.lm import lm_ops
@@ -104,6 +105,7 @@ ATTENTION = {
 LINEAR = {
     "unequal sizes": lightning(heads=3, dim=40, vdim=72),
     "one head": lightning(heads=1, dim=64, vdim=16, decay=[0.9]),
+    "decays 0 and 1": lightning(heads=2, dim=32, vdim=64, decay=[0.0, 1.0]),
     "128 / 128": lightning(heads=2, dim=128, vdim=128, decay=[0.999, 0.6]),
     "256 / 200": lightning(heads=2, dim=256, vdim=200, decay=[1.0, 0.97]),
 }
