@@ -1,10 +1,11 @@
 """ctypes binding of the engine's layer kernels (include/omniserve_lm.h), one library per element type.
 
-`lm_ops(dtype)` loads the library of torch.bfloat16 or torch.float32, building it first when the checkout holds no current one.
-There is no CPU fallback: tensors must live on the GPU."""
+`lm_ops(dtype)` loads the library of torch.bfloat16 or torch.float32, building it first when the checkout holds none (after a change
+to a source: `python -m omniserve_amd.build`).  There is no CPU fallback: tensors must live on the GPU."""
 from __future__ import annotations
 
 import ctypes
+import os
 import threading
 
 import torch
@@ -66,7 +67,8 @@ class LmOps:
             raise ValueError("no layer kernels for %s (bfloat16 and float32 have them)" % dtype)
         from .. import build
         self.dtype = dtype
-        h = _c.CDLL(build.build_lm(ELEM[dtype]))
+        path = build.lm_lib_path(ELEM[dtype])
+        h = _c.CDLL(path if os.path.exists(path) else build.build_lm(ELEM[dtype]))
         for name, (res, args) in PROTOTYPES.items():
             fn = getattr(h, name)
             fn.restype, fn.argtypes = res, args

@@ -109,16 +109,16 @@ __global__ __launch_bounds__(PT) void gelu_kernel(half_t* __restrict__ out, cons
   if constexpr (FAST) {
     v8h a, b;
 #pragma unroll
-    for (int e = 0; e < VT; ++e) { a[e] = (half_t)((float)x[e] * 0.79788456f); b[e] = (half_t)(0.044715f * (float)x[e]); }
+    for (int e = 0; e < VT; ++e) { a[e] = (half_t)rounded_f32((float)x[e] * 0.79788456f); b[e] = (half_t)rounded_f32(0.044715f * (float)x[e]); }
     u = a * ((half_t)1.0f + b * x);
   } else {
     const v8h x3 = (x * x) * x;
     v8h k;
 #pragma unroll
-    for (int e = 0; e < VT; ++e) k[e] = (half_t)(0.044715f * (float)x3[e]);
+    for (int e = 0; e < VT; ++e) k[e] = (half_t)rounded_f32(0.044715f * (float)x3[e]);
     const v8h inner = x + k;
 #pragma unroll
-    for (int e = 0; e < VT; ++e) u[e] = (half_t)(0.79788456f * (float)inner[e]);
+    for (int e = 0; e < VT; ++e) u[e] = (half_t)rounded_f32(0.79788456f * (float)inner[e]);
   }
   v8h th;
 #pragma unroll

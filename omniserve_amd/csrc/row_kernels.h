@@ -87,7 +87,7 @@ struct SrcSlabAddT {  // residual += h(GEMM epilogue(sum of split-K slabs)), in 
         ep = (half_t)(t - c);
       } else {
         const float sc = (float)r.sw[e] * sa;
-        ep = (half_t)((float)acc * sc);
+        ep = (half_t)rounded_f32((float)acc * sc);
       }
       o[e] = (half_t)((float)r.a[e] + (float)ep);
       x[e] = (float)o[e];

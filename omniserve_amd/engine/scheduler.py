@@ -112,6 +112,8 @@ class Scheduler:
             self.cache.reserve(seq, n)
             plan.append((r, n))
             budget -= n
+        if not plan and self.waiting and not self.running:
+            raise RuntimeError("no request can start: other sequences hold every slot or page")
         if not plan and self.running:
             # several unfinished prompts hold all pages: the youngest gives way
             if len(self.running) > 1:

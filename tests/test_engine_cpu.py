@@ -130,6 +130,16 @@ def test_a_request_larger_than_the_cache_is_an_error():
         e.generate([[1] * 100], SamplingParams(max_tokens=1))
 
 
+def test_sequences_of_the_caller_may_leave_no_room():
+    e = engine(None, max_tokens=256, max_seqs=1)
+    s = e.open()
+    with pytest.raises(RuntimeError, match="no request can start"):
+        e.generate([[1]])
+    e.close(s)
+    while e.has_work():
+        e.step()
+
+
 def test_stop_tokens_abort_and_bad_requests():
     e = engine(None, max_tokens=1024, max_seqs=2)
     first = e.model.expected([3, 4], 1)[0]

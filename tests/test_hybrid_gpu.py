@@ -198,7 +198,7 @@ def test_far_key_of_the_recurrent_state(dtype):
 # ---------------------------------------------------------------------------------------------------------------
 @pytest.mark.parametrize("dtype", DTYPES, ids=str)
 @pytest.mark.parametrize("tokens", [1, 7, 16, 33, 64, 65, 300, 1200])
-@pytest.mark.parametrize("kind", [dict(), dict(top=1, shared=None), dict(experts=5, top=5, ff=130, shared=16), dict(experts=70, top=8)], ids=str)
+@pytest.mark.parametrize("kind", [dict(), dict(top=1, shared=None), dict(experts=1, top=1, ff=64, shared=64), dict(experts=5, top=5, ff=130, shared=16), dict(experts=70, top=8)], ids=str)
 def test_mixture(kind, tokens, dtype):
     from omniserve_amd.backend.lm import lm_ops
     from omniserve_amd.models import layers as L
@@ -241,6 +241,55 @@ def test_residual_norm(kind, width, dtype):
     assert errors(xs[:, :width].cpu().numpy(), new).max() < 1e-6
     assert errors(h[:, :width].float().cpu().numpy(), f(new, 1)).max() < (2e-5 if dtype == F32 else 5e-3)
     assert not h[:, width:].any()
+
+
+@pytest.mark.parametrize("dtype", DTYPES, ids=str)
+@pytest.mark.parametrize("H,G,dk,dv,dims", [(4, 2, 64, 128, 64), (3, 3, 128, 64, 6), (2, 1, 256, 64, 256), (2, 2, 64, 64, 0)])
+def test_rotation_and_append(H, G, dk, dv, dims, dtype):
+    """q turned in place, k turned and v mixed into their page places; slot -1 stores nothing; far positions"""
+    from omniserve_amd.backend.lm import lm_ops
+    ops, T, g = lm_ops(dtype), 9, np.random.default_rng(23)
+    pos, slot = np.array([0, 1, 2, 63, 64, 65, 500, 4095, 100]), np.array([0, 1, 2, 63, 64 * 3, 64 * 3 + 1, 130, 64 * 2 - 1, -1])
+    x = torch.from_numpy(g.standard_normal((T, (H + G) * dk + G * dv))).to(DEV, dtype)
+    vf = torch.from_numpy(g.standard_normal((T, G * dv))).to(DEV, dtype)
+    q, k, v = (t.double().cpu().numpy() for t in x.split([H * dk, G * dk, G * dv], dim=1))
+    fr = hybrid.rope_frequencies(dims, 20000.0, dict(factor=4.0, low=1.0, high=4.0, original=300))
+    kc, vc = (torch.full((4, G, 64, d), 9.0, dtype=dtype, device=DEV) for d in (dk, dv))
+    i32 = lambda a: torch.from_numpy(a.astype(np.int32)).to(DEV)      # noqa: E731
+    ops.rope_append(x, vf, 0.3, torch.tensor(fr, dtype=F32, device=DEV), i32(pos), i32(slot), kc, vc, H, G, dk, dv)
+    tol = 3e-4 if dtype == F32 else 5e-3                                 # (angles are f32: 4095 * 2^-24)
+    turn = lambda a, n: hybrid.rotate_pairs(a.reshape(T, n, dk), pos, fr)                              # noqa: E731
+    assert errors(x[:, :H * dk].double().cpu().numpy(), turn(q, H).reshape(T, -1)).max() < tol
+    wk, wv = turn(k, G), hybrid.mix_values(v, vf.double().cpu().numpy(), 0.3).reshape(T, G, dv)
+    kn, vn = (c.double().cpu().numpy() for c in (kc, vc))
+    for t in range(T - 1):
+        p, o = divmod(slot[t], 64)
+        assert errors(kn[p, :, o], wk[t]).max() < tol and errors(vn[p, :, o], wv[t]).max() < tol
+    assert (kn == 9.0).sum() == kn.size - (T - 1) * G * dk and (vn == 9.0).sum() == vn.size - (T - 1) * G * dv
+
+
+@pytest.mark.parametrize("dtype", DTYPES, ids=str)
+@pytest.mark.parametrize("n", [40, 64, 900, 4096])
+def test_gated_rms(n, dtype):
+    from omniserve_amd.backend.lm import lm_ops
+    from omniserve_amd.models.layers import pad64, padded
+    ops, T, C, g = lm_ops(dtype), 6, pad64(n), np.random.default_rng(24)
+    o, z = (torch.from_numpy(g.standard_normal((T, n)) * s).to(dtype) for s in (1e-3, 2.0))
+    w = torch.from_numpy(1 + 0.3 * g.standard_normal(n)).float()
+    want = hybrid.rms_norm(o.double().numpy(), w.double().numpy(), 1e-6) * hybrid.sigmoid(z.double().numpy())
+    out = padded(o, T, C).to(DEV)
+    ops.gated_rms(out, out, padded(z, T, C).to(DEV), padded(w, C).to(DEV), n, 1e-6)
+    assert errors(out[:, :n].float().cpu().numpy(), want).max() < (2e-6 if dtype == F32 else 4e-3) and not out[:, n:].any()
+
+
+def test_argmax_takes_the_first_of_equals():
+    from omniserve_amd.backend.lm import lm_ops
+    z = torch.zeros((4, 5000), device=DEV)
+    z[0, 4999] = z[0, 3000] = 2.0
+    z[1] = -1.0
+    z[2, 1023] = z[2, 1024] = 1.0
+    z[3, 4200] = 9.0
+    assert lm_ops(F32).argmax(z, 4200).tolist() == [3000, 0, 1023, 0]
 
 
 @pytest.mark.parametrize("dtype", DTYPES, ids=str)
@@ -372,6 +421,17 @@ def test_unequal_requests_in_one_batch(graphs, dtype):
                 engine.close(live.pop(i)[0])
     for i, (t, ref) in enumerate(reqs):
         check(np.concatenate(got[i]), ref, dtype, "request %d" % i)
+
+
+@pytest.mark.parametrize("first", [1, 2, 70])
+def test_a_used_slot_starts_from_zero(first):
+    """whatever a slot's state holds, a new sequence's first step does not see it -- a single token, a short or a long portion"""
+    from omniserve_amd.engine import Engine
+    cfg, model, tokens, (want, _) = model_and_oracle("recurrent only", F32)
+    engine = Engine(model, max_tokens=1024, max_seqs=1)
+    for s in engine.cache.state:
+        s.fill_(float("nan"))
+    check(run_alone(engine, tokens[:140], [first, 1, 64]), want[:140], F32)
 
 
 def test_wanted_rows_come_in_the_order_asked_for():
