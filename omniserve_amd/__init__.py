@@ -1,4 +1,4 @@
-"""omniserve_amd -- MI355X (gfx950) implementation of the OmniServe quantized-inference hot path.
+"""omniserve_amd -- MI355X (gfx950) implementation of the OmniServe quantized-inference hot path, and a serving engine.
 
 Layout:
   csrc/      hand-written HIP kernels + the C ABI (include/omniserve_hip.h)
@@ -7,5 +7,8 @@ Layout:
              (same module names, function names and positional arguments)
   runtime.py minimal decode-step driver that wires the kernels like
              omniserve/modeling/models/llama_w4a8_unpad.py:406-438 (used by bench.py / smoke)
+  engine/    serving engine: paged cache and state slots, batches, scheduler, sampler
+  models/    registry and the models the engine runs (kernels: csrc/lm/, include/omniserve_lm.h, backend/lm.py)
+  cli.py     python -m omniserve_amd; trace.py: bin/trace_run
 """
 __version__ = "0.1.0"

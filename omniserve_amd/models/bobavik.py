@@ -46,7 +46,7 @@ class Bobavik(Decoder):
         dtype = dtype or torch.bfloat16
         w = Weights(state, torch.device(device), dtype)
         model = cls(parse_config(config), w, lm_ops(dtype))
-        left = w.leftovers(optional=(".mix.vmix",))        # (the first value-mixing layer carries an unused one)
+        left = w.leftovers(optional=(".mix.vmix",))        # (the layer whose values the others mix in has no use for one)
         if left:
             warnings.warn("the checkpoint has tensors the model does not use: %s" % ", ".join(left[:8]))
         return model

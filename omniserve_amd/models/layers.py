@@ -36,7 +36,7 @@ class AttentionSpec:
     dim: int
     vdim: int
     scale: float
-    window: Optional[int] = None      # a token sees itself and the window - 1 tokens before it
+    window: Optional[int] = None      # newest positions a token attends to, its own included; None: all
     rotary: Optional[RotarySpec] = None
     value_mix: bool = False           # blend the values with those of the model's first value-mixing layer
     gate: bool = True                 # sigmoid(W_g h) on the heads' output

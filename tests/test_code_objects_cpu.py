@@ -137,3 +137,28 @@ def test_midm_kernels_touch_m0_only_in_their_own_dma_statements(objects):
                         "%s: LDS-DMA without an M0 write right in front of it: %s" % (name, prev + [l])
             checked += 1
     assert checked >= 8, "expected the mid-M instantiations of all three GEMM flavours, found %d" % checked
+
+
+def test_bf16_layer_kernels_of_the_engine_do_not_spill():
+    """(heads of 256 keys and values: ten registers of the prefill attention, pinned)"""
+    import glob
+    from omniserve_amd import build as b
+    pattern = os.path.join(b.LM_CSRC, "build", "bf16", "*.o")
+    if not glob.glob(pattern):
+        b.build_lm("bf16", force=True)
+    seen = 0
+    with tempfile.TemporaryDirectory() as tmp:
+        for o in sorted(glob.glob(pattern)):
+            c = co.extract(o, tmp)
+            for k in co.kernels(c):
+                seen += 1
+                limit = 12 if "attn_prefill_kernelILi256ELi256E" in k["name"] else 0
+                assert k["spill"] <= limit, "%s: %s spills %d VGPRs" % (os.path.basename(o), k["name"], k["spill"])
+            text = co.disassemble(c)
+            assert not re.search(r"v_pk_(add|mul|fma)_f32", text), "%s: packed f32 instruction" % os.path.basename(o)
+    assert seen > 40
+
+
+def test_no_packed_f32_instruction_is_shipped(objects):
+    for tu, _, disasm in objects:
+        assert not re.search(r"v_pk_(add|mul|fma)_f32", disasm), tu
