@@ -38,7 +38,8 @@ FLAGS = ["--offload-arch=" + ARCH, "-O3", "-std=c++17", "-fPIC", "-ffp-contract=
          "-Wno-inline-asm", "-I" + CSRC, "-I" + INCLUDE]
 
 LM_CSRC = os.path.join(CSRC, "lm")
-LM_SOURCES = ["lm_rows.hip", "lm_gemm.hip", "lm_route.hip", "lm_attn.hip", "lm_attn_decode.hip", "lm_linear_attn.hip"]
+LM_SOURCES = ["lm_rows.hip", "lm_gemm.hip", "lm_route.hip", "lm_attn.hip", "lm_attn_decode.hip", "lm_linear_attn.hip",
+              "lm_latent.hip", "lm_gla.hip", "lm_delta.hip"]
 LM_FLAGS = ["--offload-arch=" + ARCH, "-O3", "-std=c++17", "-fPIC", *NO_PACKED_F32, "-Wall", "-Wno-unused-function",
             "-I" + LM_CSRC, "-I" + INCLUDE]
 LM_ELEM = {"bf16": 0, "f32": 1}        # -DLM_ELEM=<n>

@@ -40,4 +40,35 @@ __device__ __forceinline__ float softmax_step(const f32x4 (&x)[NBLK], float scal
   return alpha;
 }
 
+// Parts [B][H][nsplit][2 + dv] (maximum, sum, weighted values) of decode attention -> [B][H][dv].  One workgroup per (sequence,
+// head); at most 64 parts: lane s of every wave holds the maximum and sum of part s.
+static __global__ __launch_bounds__(256) void attn_merge_kernel(const float* part, int nsplit, const int* pos, const elem_t* gate,
+                                                                int64_t ldg, elem_t* o, int64_t ldo, int H, int dv) {
+  const int b = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63;
+  if (pos[b] < 0) return;
+  const float* q = part + ((int64_t)b * H + h) * nsplit * (dv + 2);
+  const int64_t step = dv + 2;
+  const bool in = lane < nsplit;
+  const float ms = in ? q[lane * step] : NEG, ls = in ? q[lane * step + 1] : 0.f;
+  float m = ms;
+#pragma unroll
+  for (int k = 32; k > 0; k >>= 1) m = fmaxf(m, __shfl_xor(m, k, 64));
+  const float f = __builtin_amdgcn_exp2f(ms - m), inv = 1.0f / wave_sum(f * ls);
+  for (int d0 = 0; d0 < dv; d0 += 256) {
+    const int d = d0 + threadIdx.x;
+    float y = 0.f;
+    for (int s0 = 0; s0 < nsplit; s0 += 8) {
+      float v[8];
+#pragma unroll
+      for (int s = 0; s < 8; ++s) v[s] = d < dv && s0 + s < nsplit ? q[(s0 + s) * step + 2 + d] : 0.f;
+#pragma unroll
+      for (int s = 0; s < 8; ++s) y += __shfl(f, s0 + s, 64) * v[s];
+    }
+    if (d >= dv) continue;
+    y *= inv;
+    if (gate) y *= sigmoid((float)gate[(int64_t)b * ldg + (int64_t)h * dv + d]);
+    o[(int64_t)b * ldo + (int64_t)h * dv + d] = (elem_t)y;
+  }
+}
+
 }  // namespace lm

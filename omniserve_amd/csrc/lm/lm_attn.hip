@@ -9,7 +9,8 @@ namespace lm {
 
 struct AttnArgs {
   const elem_t* q; int64_t ldq;                // [tokens][H][dk]
-  const elem_t* kc; const elem_t* vc;          // [pages][G][64][dk | dv]
+  const elem_t* kc; int64_t k_page; int k_head, k_row;      // key i of head g in page p: kc + p k_page + g k_head + i k_row
+  const elem_t* vc; int64_t v_page; int v_head, v_row;
   const int* bt; int bt_stride;                // page numbers, one row per entry
   const int* entry;                            // [entries][4]: first token, tokens, position of the first token, block table row
   const int* tiles; int n_tiles;               // [n_tiles][2]: entry, first row within the entry
@@ -62,27 +63,25 @@ __global__ __launch_bounds__(64 * WAVES, attn_waves_per_simd(DK, DV)) void attn_
 
   const int lo = max(0, pos0 + row0 - p.window + 1);     // first key the workgroup needs
   const int kb0 = lo & ~(PAGE - 1);
+  const int k_rowb = p.k_row * (int)sizeof(elem_t), v_rowb = p.v_row * (int)sizeof(elem_t);
+  // 1-KiB pieces of a tile, one per wave and turn; physical slot s of row r holds logical slot s ^ swizzle(r)
+  auto bring = [&](auto tile, const uint8_t* src, int rowb, uint8_t* dst) {
+    typedef decltype(tile) T;
+    constexpr int ROWB = T::NS * 16, N = PAGE * ROWB / 1024, STEP = 1024 * WAVES / ROWB;
+    constexpr bool EVEN = 1024 * WAVES % ROWB == 0 && STEP % 16 == 0;      // every turn's rows have the first one's swizzles
+#pragma unroll
+    for (int i = 0; i < (N + WAVES - 1) / WAVES; ++i) {
+      const int pc = wave + WAVES * i;
+      if (N % WAVES != 0 && pc >= N) continue;
+      const int sl = (EVEN ? wave : pc) * 64 + lane, r = sl / T::NS, s = sl % T::NS;
+      const uint32_t off = r * rowb + ((s ^ T::swizzle(r)) << 4);
+      dma16(src + (EVEN ? i * STEP * rowb : 0) + off, dst + 1024 * pc);
+    }
+  };
   auto stage = [&](int kb, uint8_t* kt, uint8_t* vt) {
     const int64_t page = bt[kb / PAGE];
-    const uint8_t* ks = (const uint8_t*)(p.kc + (page * p.G + g) * (PAGE * DK));
-    const uint8_t* vs = (const uint8_t*)(p.vc + (page * p.G + g) * (PAGE * DV));
-    constexpr int KP = PAGE * Gm::KB / 1024, VP = PAGE * Gm::VB / 1024;      // 1-KiB pieces
-#pragma unroll
-    for (int i = 0; i < (KP + WAVES - 1) / WAVES; ++i) {
-      const int pc = wave + WAVES * i;
-      if (KP % WAVES == 0 || pc < KP) {
-        const int sl = pc * 64 + lane, r = sl / KT::NS, s = sl % KT::NS;
-        dma16(ks + KT::slot(r, s), kt + 1024 * pc);      // physical slot s of row r holds logical slot s ^ swizzle(r)
-      }
-    }
-#pragma unroll
-    for (int i = 0; i < (VP + WAVES - 1) / WAVES; ++i) {
-      const int pc = wave + WAVES * i;
-      if (VP % WAVES == 0 || pc < VP) {
-        const int sl = pc * 64 + lane, r = sl / VT::NS, s = sl % VT::NS;
-        dma16(vs + VT::slot(r, s), vt + 1024 * pc);
-      }
-    }
+    bring(KT{}, (const uint8_t*)(p.kc + page * p.k_page + g * p.k_head), k_rowb, kt);
+    bring(VT{}, (const uint8_t*)(p.vc + page * p.v_page + g * p.v_head), v_rowb, vt);
   };
   auto compute = [&](int kb, const uint8_t* kt, const uint8_t* vt, auto prefetch) {
     const bool skip = idle || kb > w_last || kb + PAGE - 1 <= w_first - p.window;      // nothing visible for this wave
@@ -179,18 +178,20 @@ static int launch(const AttnArgs& a, hipStream_t s) {
 
 using namespace lm;
 
-extern "C" int lm_attn_prefill(const void* q, int64_t ldq, const void* kc, const void* vc, const int* bt, int bt_stride,
-                               const int* entry, const int* tiles, int n_tiles, const void* gate, int64_t ldg, void* o, int64_t ldo,
+extern "C" int lm_attn_prefill(const void* q, int64_t ldq, const void* kc, int64_t k_page, int k_head, int k_row,
+                               const void* vc, int64_t v_page, int v_head, int v_row, const int* bt, int bt_stride, const int* entry, const int* tiles, int n_tiles, const void* gate, int64_t ldg, void* o, int64_t ldo,
                                float scale, int window, int H, int G, int dk, int dv, void* stream) {
   if (n_tiles <= 0 || G <= 0 || H % G || !(scale > 0.f) || window <= 0 || ldq % FR || ldo % 4 || ldg % 4 ||
+      k_page % FR || k_head % FR || k_row % FR || v_page % FR || v_head % FR || v_row % FR ||
+      k_row <= 0 || v_row <= 0 || k_row > (1 << 22) || v_row > (1 << 22) ||
       (int64_t)n_tiles * H > (1 << 28))
     return LM_EINVAL;
-  AttnArgs a{(const elem_t*)q, ldq, (const elem_t*)kc, (const elem_t*)vc, bt, bt_stride, entry, tiles, n_tiles, (const elem_t*)gate,
+  AttnArgs a{(const elem_t*)q, ldq, (const elem_t*)kc, k_page, k_head, k_row, (const elem_t*)vc, v_page, v_head, v_row, bt, bt_stride, entry, tiles, n_tiles, (const elem_t*)gate,
              ldg, (elem_t*)o, ldo, scale * 1.4426950408889634f, window, H, G};
   hipStream_t s = (hipStream_t)stream;
 #define LM_CASE(K, V) if (dk == K && dv == V) return launch<K, V>(a, s);
   LM_CASE(64, 64) LM_CASE(64, 128) LM_CASE(64, 256) LM_CASE(128, 64) LM_CASE(128, 128) LM_CASE(128, 256)
-  LM_CASE(256, 64) LM_CASE(256, 128) LM_CASE(256, 256)
+  LM_CASE(192, 64) LM_CASE(192, 128) LM_CASE(192, 256) LM_CASE(256, 64) LM_CASE(256, 128) LM_CASE(256, 256)
 #undef LM_CASE
   return LM_EINVAL;
 }

@@ -191,34 +191,6 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(DecodeArgs p) {
   }
 }
 
-// one workgroup per (sequence, head); at most 64 parts: lane s of every wave holds the maximum and sum of part s
-__global__ __launch_bounds__(256) void attn_merge_kernel(const float* part, int nsplit, const int* pos, const elem_t* gate, int64_t ldg,
-                                                         elem_t* o, int64_t ldo, int H, int dv) {
-  const int b = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63;
-  if (pos[b] < 0) return;
-  const float* q = part + ((int64_t)b * H + h) * nsplit * (dv + 2);
-  const int64_t step = dv + 2;
-  const bool in = lane < nsplit;
-  const float ms = in ? q[lane * step] : NEG, ls = in ? q[lane * step + 1] : 0.f;
-  float m = ms;
-#pragma unroll
-  for (int k = 32; k > 0; k >>= 1) m = fmaxf(m, __shfl_xor(m, k, 64));
-  const float f = __builtin_amdgcn_exp2f(ms - m), inv = 1.0f / wave_sum(f * ls);
-  const int d = threadIdx.x;
-  float y = 0.f;
-  for (int s0 = 0; s0 < nsplit; s0 += 8) {
-    float v[8];
-#pragma unroll
-    for (int s = 0; s < 8; ++s) v[s] = d < dv && s0 + s < nsplit ? q[(s0 + s) * step + 2 + d] : 0.f;
-#pragma unroll
-    for (int s = 0; s < 8; ++s) y += __shfl(f, s0 + s, 64) * v[s];
-  }
-  if (d >= dv) return;
-  y *= inv;
-  if (gate) y *= sigmoid((float)gate[(int64_t)b * ldg + (int64_t)h * dv + d]);
-  o[(int64_t)b * ldo + (int64_t)h * dv + d] = (elem_t)y;
-}
-
 template <int DK, int DV>
 static int launch(const DecodeArgs& a, int B, hipStream_t s) {
   const int gs = a.H / a.G, hb = (gs + 15) / 16;

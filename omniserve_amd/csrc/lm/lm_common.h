@@ -82,6 +82,15 @@ __device__ __forceinline__ void split_quad(f32x4 x, quad_t (&q)[NOPND]) {
 
 __device__ __forceinline__ float sigmoid(float z) { return __builtin_amdgcn_rcpf(1.0f + __expf(-z)); }      // (rcp: within an ulp)
 __device__ __forceinline__ float silu(float z) { return z * sigmoid(z); }
+__device__ __forceinline__ float gelu_tanh(float z) {      // 0.5 z (1 + tanh u) = z sigmoid(2 u)
+  return z * sigmoid(1.5957691216057308f * (z + 0.044715f * z * z * z));
+}
+// log(1 + e^z)
+__device__ __forceinline__ float softplus(float z) {
+  const float e = __expf(-fabsf(z)), u = 1.0f + e, d = u - 1.0f;
+  return fmaxf(z, 0.f) + (d == 0.f ? e : __logf(u) * e * __builtin_amdgcn_rcpf(d));      // log1p(e) without the cancellation
+}
+constexpr float LOG2E = 1.4426950408889634f;
 
 // lam^n for n >= 0, from log2(lam)
 __device__ __forceinline__ float power(float log2_lam, int n) { return n == 0 ? 1.0f : __builtin_amdgcn_exp2f((float)n * log2_lam); }
@@ -109,9 +118,9 @@ __device__ __forceinline__ float column_sum(float v) {
 template <int ROWB>
 struct Tile {
   static constexpr int NS = ROWB / 16;
-  static_assert(NS >= 8 && (NS & (NS - 1)) == 0, "row size");
+  static_assert(NS >= 8 && NS % 8 == 0, "row size");
   __device__ __forceinline__ static int swizzle(int row) {
-    if constexpr (NS == 8) {         // neighbouring rows share a line
+    if constexpr (NS / 8 % 2 == 1) { // an odd number of half lines: neighbouring rows start in different halves
       const int q = (row >> 1) & 7;
       return (((q ^ ((q >> 1) & 2)) & 3) << 1) | (q >> 2);
     }

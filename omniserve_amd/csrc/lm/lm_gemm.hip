@@ -5,8 +5,8 @@
 //                  once; its waves split K and meet in LDS.  Weights are the A operand straight from global memory.
 //   lm_gemm_tiles  many rows (prefill): MFMA bound.  256 x 128 tiles, both operands by LDS-DMA, two stages ahead.
 //
-// Epilogues: element type, f32 times a factor, or the gated unit silu(gate) * up of a matrix whose rows alternate in blocks of
-// 16 between gate and up channels (both halves of a pair then sit in the same lane).
+// Epilogues: element type, f32 times a factor, the gated unit act(gate + bias) * (up + bias) of a matrix whose rows alternate in
+// blocks of 16 between gate and up channels (both halves of a pair then sit in the same lane), or the product with sigmoid(gate).
 #include "lm_common.h"
 #include "omniserve_lm.h"
 
@@ -17,6 +17,10 @@ struct Part {        // a family of equally shaped groups
   const elem_t* x; int64_t ldx;
   void* y; int64_t ldy;
   int n, k;
+  int64_t gx, gy;            // without perm: columns of x / y between neighbouring groups
+  const float* bias;         // [n] added to the products of a gated unit (or null)
+  const elem_t* gate;        // LM_EPI_GATE: the factor's argument, laid out like y
+  int64_t ldg;
 };
 
 struct GemmArgs {
@@ -28,19 +32,36 @@ struct GemmArgs {
   int x_div;                  // x row = y row / x_div (tokens of (token, choice) pairs)
   const int* tiles;           // lm_gemm_tiles with perm: (group, first place, rows, 0) of every row tile, rows 0: none
   float scale;
+  int act;                    // of the gated unit
 };
 
-template <int EPI>
-__device__ __forceinline__ void store4(const Part& pt, int64_t row, int c, f32x4 v, f32x4 up, float scale) {
-  if constexpr (EPI == LM_EPI_ELEM) {
-    *(quad_t*)((elem_t*)pt.y + row * pt.ldy + c) = to_quad(v);
-  } else if constexpr (EPI == LM_EPI_F32) {
-    *(f32x4*)((float*)pt.y + row * pt.ldy + c) = v * scale;
-  } else {
-    f32x4 r;
+__device__ __forceinline__ f32x4 glu(const Part& pt, int act, int c, f32x4 gate, f32x4 up) {      // c: gate channel's row in w, a multiple of 4
+  if (pt.bias) {
+    gate += *(const f32x4*)(pt.bias + c);
+    up += *(const f32x4*)(pt.bias + c + 16);
+  }
+  f32x4 r;
+  if (act == LM_ACT_GELU_TANH) {
 #pragma unroll
-    for (int e = 0; e < 4; ++e) r[e] = silu(v[e]) * up[e];
-    *(quad_t*)((elem_t*)pt.y + row * pt.ldy + c) = to_quad(r);
+    for (int e = 0; e < 4; ++e) r[e] = gelu_tanh(gate[e]) * up[e];
+  } else {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) r[e] = silu(gate[e]) * up[e];
+  }
+  return r;
+}
+
+template <int EPI>
+__device__ __forceinline__ void store4(const Part& pt, int64_t row, int c, int64_t y0, f32x4 v, float scale) {
+  if constexpr (EPI == LM_EPI_ELEM || EPI == LM_EPI_GLU) {
+    *(quad_t*)((elem_t*)pt.y + row * pt.ldy + y0 + c) = to_quad(v);
+  } else if constexpr (EPI == LM_EPI_F32) {
+    *(f32x4*)((float*)pt.y + row * pt.ldy + y0 + c) = v * scale;
+  } else {
+    const f32x4 z = from_quad(*(const quad_t*)(pt.gate + row * pt.ldg + y0 + c));
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] *= sigmoid(z[e]);
+    *(quad_t*)((elem_t*)pt.y + row * pt.ldy + y0 + c) = to_quad(v);
   }
 }
 
@@ -60,6 +81,7 @@ __global__ __launch_bounds__(64 * KW) void gemm_rows_kernel(GemmArgs p) {
   if (perm) { first = p.off[g]; rows = p.off[g + 1] - first; }
   if (rows <= 0) return;
   const elem_t* w = pt.w + (is_b ? 0 : (int64_t)g * pt.n * pt.k);
+  const int64_t x0 = is_b || perm ? 0 : g * pt.gx, y0 = is_b || perm ? 0 : g * pt.gy;
   const int steps = pt.k / KSTEP, s0 = steps * wave / KW, s1 = steps * (wave + 1) / KW;
   const elem_t* wp[NR];
 #pragma unroll
@@ -74,7 +96,7 @@ __global__ __launch_bounds__(64 * KW) void gemm_rows_kernel(GemmArgs p) {
     for (int m = 0; m < MB; ++m) {
       const int i = m0 + 16 * m + l15, ic = i < rows ? i : rows - 1;
       const int pair = perm ? perm[first + ic] : ic;
-      xp[m] = pt.x + (int64_t)(pair / div) * pt.ldx + FR * l4;
+      xp[m] = pt.x + (int64_t)(pair / div) * pt.ldx + x0 + FR * l4;
     }
     const int mb = min(MB, (rows - m0 + 15) >> 4);     // row blocks with work (uniform)
     f32x4 acc[NR][MB];
@@ -160,7 +182,10 @@ __global__ __launch_bounds__(64 * KW) void gemm_rows_kernel(GemmArgs p) {
       }
       const int pair = perm ? perm[first + m0 + m] : m0 + m;
       const int c = (EPI == LM_EPI_GLU ? n0 / 2 : n0) + 16 * blk + c4;
-      if (c < (EPI == LM_EPI_GLU ? pt.n / 2 : pt.n)) store4<EPI>(pt, pair, c, v, up, p.scale);
+      if (c < (EPI == LM_EPI_GLU ? pt.n / 2 : pt.n)) {
+        if constexpr (EPI == LM_EPI_GLU) v = glu(pt, p.act, n0 + 16 * sb + c4, v, up);
+        store4<EPI>(pt, pair, c, y0, v, p.scale);
+      }
     }
     __syncthreads();
   }
@@ -285,7 +310,7 @@ __global__ __launch_bounds__(256, 2) void gemm_tiles_kernel(GemmArgs p, int mt_a
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int c = n0 + wn + 16 * i + 4 * l4;
-        if (c < pt.n) store4<EPI>(pt, row, c, acc[i][j], zero4(), p.scale);
+        if (c < pt.n) store4<EPI>(pt, row, c, 0, acc[i][j], p.scale);
       }
     }
   } else {
@@ -304,8 +329,7 @@ __global__ __launch_bounds__(256, 2) void gemm_tiles_kernel(GemmArgs p, int mt_a
           int c = 16 * i;
           if constexpr (EPI == LM_EPI_GLU) {
             c = 8 * i;
-#pragma unroll
-            for (int e = 0; e < 4; ++e) v[e] = silu(v[e]) * acc[i + 1][j][e];
+            if (n0 + wn + 16 * i < pt.n) v = glu(pt, p.act, n0 + wn + 16 * i + 4 * l4, v, acc[i + 1][j]);
           }
           *(quad_t*)(buf + (16 * jj + l15) * PITCH + (c + 4 * l4) * (int)sizeof(elem_t)) = to_quad(v);
         }
@@ -325,23 +349,26 @@ __global__ __launch_bounds__(256, 2) void gemm_tiles_kernel(GemmArgs p, int mt_a
   }
 }
 
-static int check_part(const Part& p, int epi) {
+static int check_part(const Part& p, int epi, int act) {
   if (!p.w || !p.x || !p.y || p.n <= 0 || p.k <= 0 || p.k % 64 || p.n % 16 || p.ldx < p.k || p.ldx % FR || p.ldy % FR) return LM_EINVAL;
-  if (epi == LM_EPI_GLU && p.n % 32) return LM_EINVAL;
+  if (epi == LM_EPI_GLU && (p.n % 32 || (act != LM_ACT_SILU && act != LM_ACT_GELU_TANH))) return LM_EINVAL;
+  if (epi == LM_EPI_GATE && (!p.gate || p.ldg % 4)) return LM_EINVAL;
+  if (p.gx % FR || p.gy % 4) return LM_EINVAL;
   return LM_OK;
 }
 
 static int fill(GemmArgs& a, const LmGemmPart* pa, const LmGemmPart* pb, int groups, const int* perm, const int* off, int rows_a,
-                int rows_b, int x_div, float scale, int epi) {
+                int rows_b, int x_div, float scale, int epi, int act) {
   auto conv = [](const LmGemmPart* s) {
-    return Part{(const elem_t*)s->w, (const elem_t*)s->x, s->ldx, s->y, s->ldy, s->n, s->k};
+    return Part{(const elem_t*)s->w, (const elem_t*)s->x, s->ldx, s->y, s->ldy, s->n, s->k, s->gx, s->gy, s->bias,
+                (const elem_t*)s->gate, s->ldg};
   };
-  if (!pa || groups <= 0 || x_div <= 0 || (groups > 1 && !perm) || (perm && !off) || epi < 0 || epi > LM_EPI_GLU) return LM_EINVAL;
+  if (!pa || groups <= 0 || x_div <= 0 || (perm && !off) || epi < 0 || epi > LM_EPI_GATE) return LM_EINVAL;
   a.a = conv(pa);
   a.b = pb ? conv(pb) : Part{};
-  if (check_part(a.a, epi) || (pb && check_part(a.b, epi))) return LM_EINVAL;
+  if (check_part(a.a, epi, act) || (pb && check_part(a.b, epi, act))) return LM_EINVAL;
   a.groups = groups; a.perm = perm; a.off = off; a.rows_a = rows_a; a.rows_b = pb ? rows_b : 0; a.x_div = perm ? x_div : 1;
-  a.tiles = nullptr; a.scale = scale;
+  a.tiles = nullptr; a.scale = scale; a.act = act;
   return LM_OK;
 }
 
@@ -377,20 +404,22 @@ static int plan_rows(const GemmArgs& a, int max_rows, int has_b, hipStream_t s) 
 using namespace lm;
 
 extern "C" int lm_gemm_rows(const LmGemmPart* pa, const LmGemmPart* pb, int groups, const int* perm, const int* off, int rows_a,
-                            int rows_b, int x_div, int max_rows, float scale, int epi, void* stream) {
+                            int rows_b, int x_div, int max_rows, float scale, int epi, int act, void* stream) {
   GemmArgs a;
-  if (fill(a, pa, pb, groups, perm, off, rows_a, rows_b, x_div, scale, epi) || max_rows <= 0) return LM_EINVAL;
+  if (fill(a, pa, pb, groups, perm, off, rows_a, rows_b, x_div, scale, epi, act) || max_rows <= 0) return LM_EINVAL;
   hipStream_t s = (hipStream_t)stream;
   const int has_b = pb && rows_b > 0;
   if (epi == LM_EPI_GLU) return plan_rows<LM_EPI_GLU>(a, max_rows, has_b, s);
+  if (epi == LM_EPI_GATE) return plan_rows<LM_EPI_GATE>(a, max_rows, has_b, s);
   return epi == LM_EPI_F32 ? plan_rows<LM_EPI_F32>(a, max_rows, has_b, s) : plan_rows<LM_EPI_ELEM>(a, max_rows, has_b, s);
 }
 
 extern "C" int lm_gemm_tiles(const LmGemmPart* pa, const LmGemmPart* pb, int groups, const int* perm, const int* off,
                              const int* tiles, int max_tiles, int rows_a, int rows_b, int x_div,
-                             float scale, int epi, void* stream) {
+                             float scale, int epi, int act, void* stream) {
   GemmArgs a;
-  if (fill(a, pa, pb, groups, perm, off, rows_a, rows_b, x_div, scale, epi)) return LM_EINVAL;
+  if (fill(a, pa, pb, groups, perm, off, rows_a, rows_b, x_div, scale, epi, act)) return LM_EINVAL;
+  if (epi == LM_EPI_GATE || (groups > 1 && !perm)) return LM_EINVAL;      // few rows only
   if (perm && (!tiles || max_tiles <= 0)) return LM_EINVAL;
   a.tiles = perm ? tiles : nullptr;
   const int mt_a = perm ? max_tiles : (rows_a + TM - 1) / TM, mt_b = pb && rows_b > 0 ? (rows_b + TM - 1) / TM : 0;

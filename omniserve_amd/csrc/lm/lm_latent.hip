@@ -1,0 +1,278 @@
+// Latent attention: the cache holds one row per token, [normed latent c | turned key part], that all heads share.
+//
+//   lm_latent_append  prompt portions: norm + rotation of the row, stored in its page; the queries' turned parts in place.  (The
+//                     portions' attention runs on keys and values expanded from the rows by a product: lm_attn_prefill.)
+//   lm_latent_decode  one token per sequence: the queries' unturned parts have been taken into the latent space (W_uk^T q), so a
+//                     cache row is key (all of it) and value (its latent) of every head.  A workgroup serves 16 heads, the columns
+//                     of the MFMA tiles, and one part of the keys; its waves share the rows in LDS, form the same scores and own a
+//                     quarter of the latent's columns each, so nothing but the tiles passes between them.
+//   lm_gather_pages   the pages of the portions' contexts, one behind the other
+#include "lm_attn.h"
+#include "omniserve_lm.h"
+
+namespace lm {
+
+// The cache row of one token from its projection; the whole workgroup (256 threads), Rp <= 1024.  Both may be the same row.
+__device__ __forceinline__ void latent_row(const elem_t* src, const float* w, float eps, const float* freq, int half, int pos,
+                                           elem_t* dst, int R, int Rp, int Tp, float* red) {
+  const int tid = threadIdx.x, c = 4 * tid;
+  const f32x4 v = c < Rp ? from_quad(*(const quad_t*)(src + c)) : zero4();      // (columns from R on are zero)
+  const float ss = wave_sum((v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]));
+  if ((tid & 63) == 0) red[tid >> 6] = ss;
+  __syncthreads();
+  const float r = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)R + eps);
+  if (c < Rp) *(quad_t*)(dst + c) = to_quad(v * r * *(const f32x4*)(w + c));
+  if (tid < half) {
+    float s, co;
+    sincosf((float)pos * freq[tid], &s, &co);
+    const float a = (float)src[Rp + tid], b = (float)src[Rp + half + tid];
+    dst[Rp + tid] = (elem_t)(a * co - b * s);
+    dst[Rp + half + tid] = (elem_t)(b * co + a * s);
+  } else if (tid + half < Tp) {
+    dst[Rp + half + tid] = (elem_t)0.f;
+  }
+}
+
+struct LatentAppendArgs {
+  elem_t* x; int64_t ld, src_col;       // row: q [H][dk], ..., from src_col on the projected cache row; src_col < 0: none
+  const float* w; float eps;
+  const float* freq; int half;
+  const int *pos, *slot;
+  elem_t* cache;                        // [pages][64][Rp + Tp]
+  int H, dk, q_rot, R, Rp, Tp;
+};
+
+__global__ __launch_bounds__(256) void latent_append_kernel(LatentAppendArgs p) {
+  __shared__ f32x2 cs[128];
+  __shared__ float red[4];
+  const int t = blockIdx.x, tid = threadIdx.x, pos = p.pos[t], slot = p.slot[t];
+  if (tid < p.half) {
+    float s, c;
+    sincosf((float)pos * p.freq[tid], &s, &c);
+    cs[tid] = (f32x2){c, s};
+  }
+  __syncthreads();
+  elem_t* row = p.x + (int64_t)t * p.ld;
+  for (int i = tid; i < p.H * p.half; i += 256) {
+    const int h = i / p.half, d = i - h * p.half;
+    elem_t* q = row + (int64_t)h * p.dk + p.q_rot + d;
+    const float a = (float)q[0], b = (float)q[p.half];
+    q[0] = (elem_t)(a * cs[d][0] - b * cs[d][1]);
+    q[p.half] = (elem_t)(b * cs[d][0] + a * cs[d][1]);
+  }
+  if (p.src_col >= 0 && slot >= 0)
+    latent_row(row + p.src_col, p.w, p.eps, p.freq, p.half, pos, p.cache + (int64_t)slot * (p.Rp + p.Tp), p.R, p.Rp, p.Tp, red);
+}
+
+__global__ __launch_bounds__(256) void gather_pages_kernel(frag_t* dst, const frag_t* src, const int* pages, int row_frags) {
+  const int n = PAGE * row_frags;
+  const frag_t* s = src + (int64_t)pages[blockIdx.x] * n;
+  frag_t* d = dst + (int64_t)blockIdx.x * n;
+  for (int i = threadIdx.x + 256 * blockIdx.y; i < n; i += 256 * gridDim.y) d[i] = s[i];
+}
+
+struct LatentDecodeArgs {
+  const elem_t* x; int64_t ld, src_col;        // as above; the queries' turned parts are read as projected
+  const float* w; float eps;
+  const float* freq; int half;
+  const int *pos, *slot;                       // pos < 0: an empty place of the batch
+  elem_t* cache;
+  const int* bt; int bt_stride;
+  const elem_t* qa;                            // [B][H][RP]
+  elem_t* o;                                   // [B][H][RP]
+  float* part;                                 // nsplit > 1: [B][H][nsplit][RP + 2]
+  float scale;                                 // includes log2(e)
+  int nsplit, H, dk, q_rot, R;
+};
+
+template <int RP, int TP>
+struct LatentGeom {
+  static constexpr int KT = 32, ROW = RP + TP, ES = (int)sizeof(elem_t);
+  static constexpr int CB = KT * RP * ES, TB = KT * TP * ES, BUF = CB + TB, QB = 16 * ROW * ES;
+  static constexpr int NBUF = 2 * BUF <= 155648 ? 2 : 1;
+  static constexpr size_t LDS = NBUF * BUF > QB ? NBUF * BUF : QB;
+};
+
+template <int RP, int TP>
+__global__ __launch_bounds__(256, SPLIT ? 2 : 1) void latent_decode_kernel(LatentDecodeArgs p) {
+  typedef LatentGeom<RP, TP> Gm;
+  typedef Tile<RP * (int)sizeof(elem_t)> CT;
+  typedef Tile<TP * (int)sizeof(elem_t)> TT;
+  constexpr int ROW = Gm::ROW, NCF = RP / KSTEP, NTF = TP / KSTEP, NVB = RP / 64;
+  extern __shared__ __attribute__((aligned(16))) uint8_t lds[];      // the queries, then the key tiles
+  __shared__ float red[4];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l15 = lane & 15, l4 = lane >> 4;
+  const int b = blockIdx.x, h0 = 16 * blockIdx.y, nh = min(16, p.H - h0), split = blockIdx.z;
+  const int pos = p.pos[b];
+  if (pos < 0) return;
+  const int nt = pos / Gm::KT + 1, per = (nt + p.nsplit - 1) / p.nsplit, ta = split * per, tb = min(nt, ta + per);
+  const int* bt = p.bt + (int64_t)b * p.bt_stride;
+  const elem_t* row = p.x + (int64_t)b * p.ld;
+
+  elem_t(*qs)[ROW] = (elem_t(*)[ROW])lds;
+  for (int i = tid; i < 16 * (RP / FR); i += 256) {
+    const int hh = i / (RP / FR), d = (i - hh * (RP / FR)) * FR;
+    *(frag_t*)&qs[hh][d] = hh < nh ? *(const frag_t*)(p.qa + ((int64_t)b * p.H + h0 + hh) * RP + d) : frag_t{};
+  }
+  for (int i = tid; i < 16 * (TP / 2); i += 256) {      // pairs; those past `half` are padding
+    const int hh = i / (TP / 2), d = i - hh * (TP / 2);
+    float a = 0.f, c = 0.f;
+    if (d < p.half && hh < nh) {
+      const elem_t* q = row + (int64_t)(h0 + hh) * p.dk + p.q_rot + d;
+      const float u = (float)q[0], v = (float)q[p.half];
+      float s, co;
+      sincosf((float)pos * p.freq[d], &s, &co);
+      a = u * co - v * s;
+      c = v * co + u * s;
+    }
+    const int at = d < p.half ? d : 2 * p.half + 2 * (d - p.half);
+    qs[hh][RP + at] = (elem_t)a;
+    qs[hh][RP + (d < p.half ? d + p.half : at + 1)] = (elem_t)c;
+  }
+  // the new row: written by every workgroup that reads it itself (equal bytes), the ones whose part holds the newest tile
+  const int slot = p.slot[b];
+  if (tb == nt && ta < tb && slot >= 0 && p.src_col >= 0)
+    latent_row(row + p.src_col, p.w, p.eps, p.freq, p.half, pos, p.cache + (int64_t)slot * ROW, p.R, RP, TP, red);
+  __syncthreads();      // (also makes the appended row visible to the other waves of this workgroup)
+  frag_t qf[NCF + NTF];
+#pragma unroll
+  for (int s = 0; s < NCF + NTF; ++s) qf[s] = *(const frag_t*)&qs[l15][s * KSTEP + FR * l4];
+  f32x4 acc[NVB];
+#pragma unroll
+  for (int c = 0; c < NVB; ++c) acc[c] = zero4();
+  float m_run = NEG, l_run = 0.f;
+  __syncthreads();      // the queries' place is free
+
+  auto stage = [&](int t, uint8_t* buf) {
+    const int kb = Gm::KT * t;
+    const elem_t* src = p.cache + ((int64_t)bt[kb / PAGE] * PAGE + kb % PAGE) * ROW;
+#pragma unroll
+    for (int i = 0; i < (Gm::CB / 1024 + 3) / 4; ++i) {
+      const int pc = wave + 4 * i, sl = pc * 64 + lane, r = sl / CT::NS, s = sl % CT::NS;
+      dma16(src + r * ROW + (s ^ CT::swizzle(r)) * FR, buf + 1024 * pc);
+    }
+#pragma unroll
+    for (int i = 0; i < (Gm::TB / 1024 + 3) / 4; ++i) {
+      const int pc = wave + 4 * i, sl = pc * 64 + lane, r = sl / TT::NS, s = sl % TT::NS;
+      dma16(src + r * ROW + RP + (s ^ TT::swizzle(r)) * FR, buf + Gm::CB + 1024 * pc);
+    }
+  };
+  static_assert(Gm::CB % 4096 == 0 && Gm::TB % 4096 == 0, "whole pieces for four waves");
+  auto compute = [&](int t, const uint8_t* ct, auto prefetch) {
+    const int kb = Gm::KT * t;
+    const uint8_t* tt = ct + Gm::CB;
+    f32x4 x[2];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      x[u] = zero4();
+#pragma unroll
+      for (int s = 0; s < NCF; ++s) x[u] = mma(CT::frag(ct, 16 * u + l15, 4 * s + l4), qf[s], x[u]);
+#pragma unroll
+      for (int s = 0; s < NTF; ++s) x[u] = mma(TT::frag(tt, 16 * u + l15, 4 * s + l4), qf[NCF + s], x[u]);
+      __builtin_amdgcn_sched_barrier(0);      // (not all of the tile's operands in registers at once)
+    }
+    prefetch();
+    if (kb + Gm::KT - 1 > pos) {
+#pragma unroll
+      for (int u = 0; u < 2; ++u)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) x[u][r] = kb + 16 * u + 4 * l4 + r <= pos ? x[u][r] : NEG;
+    }
+    quad_t pq[2][NOPND];
+    const float alpha = softmax_step<2>(x, p.scale, m_run, l_run, pq);
+#pragma unroll
+    for (int c = 0; c < NVB; ++c) {
+      acc[c] *= alpha;
+      const quad_t v0 = CT::column_quad(ct, 0, wave * NVB + c, l15, l4), v1 = CT::column_quad(ct, 16, wave * NVB + c, l15, l4);
+#pragma unroll
+      for (int o = 0; o < NOPND; ++o) acc[c] = mma_quads(v0, v1, pq[0][o], pq[1][o], acc[c]);
+    }
+  };
+  if constexpr (Gm::NBUF == 2) {
+    if (ta < tb) stage(ta, lds);
+    __syncthreads();
+    for (int t = ta; t < tb; ++t) {
+      uint8_t *now = lds + ((t - ta) & 1) * Gm::BUF, *next = lds + ((t - ta + 1) & 1) * Gm::BUF;
+      compute(t, now, [&] { if (t + 1 < tb) stage(t + 1, next); });
+      __syncthreads();
+    }
+  } else {
+    for (int t = ta; t < tb; ++t) {
+      stage(t, lds);
+      __syncthreads();
+      compute(t, lds, [] {});
+      __syncthreads();
+    }
+  }
+  l_run = column_sum(l_run);
+  if (l15 >= nh) return;
+  const int64_t hrow = (int64_t)b * p.H + h0 + l15;
+  if (p.nsplit > 1) {
+    float* q = p.part + (hrow * p.nsplit + split) * (RP + 2);
+    if (wave == 0 && l4 == 0) { q[0] = m_run; q[1] = l_run; }
+#pragma unroll
+    for (int c = 0; c < NVB; ++c)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) q[2 + 16 * (wave * NVB + c) + 4 * l4 + r] = acc[c][r];
+  } else {
+    const float inv = 1.0f / l_run;
+#pragma unroll
+    for (int c = 0; c < NVB; ++c) *(quad_t*)(p.o + hrow * RP + 16 * (wave * NVB + c) + 4 * l4) = to_quad(acc[c] * inv);
+  }
+}
+
+template <int RP, int TP>
+static int launch(const LatentDecodeArgs& a, int B, hipStream_t s) {
+  typedef LatentGeom<RP, TP> Gm;
+  auto k = latent_decode_kernel<RP, TP>;
+  if (allow_lds(k, Gm::LDS)) return LM_EINVAL;
+  hipLaunchKernelGGL(k, dim3(B, (a.H + 15) / 16, a.nsplit), dim3(256), Gm::LDS, s, a);
+  if (a.nsplit > 1)
+    hipLaunchKernelGGL(attn_merge_kernel, dim3(B, a.H), dim3(256), 0, s, a.part, a.nsplit, a.pos, (const elem_t*)nullptr, (int64_t)0, a.o,
+                       (int64_t)a.H * RP, a.H, RP);
+  return launch_status();
+}
+
+static int check(int64_t ld, int64_t src_col, const float* w, int half, int H, int dk, int q_rot, int R, int Rp, int Tp) {
+  if (H <= 0 || half < 0 || 2 * half > Tp || Tp > 256 || q_rot < 0 || q_rot + 2 * half > dk || R <= 0 || R > Rp || Rp % 64 || Rp > 1024 ||
+      Tp % 64 || ld % FR || (src_col >= 0 && (!w || src_col % FR)))
+    return LM_EINVAL;
+  return LM_OK;
+}
+
+}  // namespace lm
+
+using namespace lm;
+
+extern "C" int lm_latent_append(void* x, int64_t ld, int64_t src_col, const float* w, float eps, const float* freq, int half,
+                                const int* pos, const int* slot, void* cache, int tokens, int H, int dk, int q_rot, int R, int Rp, int Tp,
+                                void* stream) {
+  if (tokens <= 0 || check(ld, src_col, w, half, H, dk, q_rot, R, Rp, Tp)) return LM_EINVAL;
+  LatentAppendArgs a{(elem_t*)x, ld, src_col, w, eps, freq, half, pos, slot, (elem_t*)cache, H, dk, q_rot, R, Rp, Tp};
+  hipLaunchKernelGGL(latent_append_kernel, dim3(tokens), dim3(256), 0, (hipStream_t)stream, a);
+  return launch_status();
+}
+
+extern "C" int lm_gather_pages(void* dst, const void* src, const int* pages, int n_pages, int row, void* stream) {
+  if (n_pages <= 0 || row <= 0 || row % FR) return LM_EINVAL;
+  hipLaunchKernelGGL(gather_pages_kernel, dim3(n_pages, 4), dim3(256), 0, (hipStream_t)stream, (frag_t*)dst, (const frag_t*)src, pages,
+                     row / FR);
+  return launch_status();
+}
+
+extern "C" int lm_latent_decode(const void* x, int64_t ld, int64_t src_col, const float* w, float eps, const float* freq, int half,
+                                const int* pos, const int* slot, void* cache, const int* bt, int bt_stride, const void* qa, void* o,
+                                float* part, int nsplit, float scale, int B, int H, int dk, int q_rot, int R, int Rp, int Tp,
+                                void* stream) {
+  if (B <= 0 || nsplit <= 0 || nsplit > 64 || (nsplit > 1 && !part) || !(scale > 0.f) ||
+      check(ld, src_col, w, half, H, dk, q_rot, R, Rp, Tp))
+    return LM_EINVAL;
+  LatentDecodeArgs a{(const elem_t*)x, ld, src_col, w, eps, freq, half, pos, slot, (elem_t*)cache, bt, bt_stride, (const elem_t*)qa,
+                     (elem_t*)o, part, scale * LOG2E, nsplit, H, dk, q_rot, R};
+  hipStream_t s = (hipStream_t)stream;
+#define LM_CASE(K, V) if (Rp == K && Tp == V) return launch<K, V>(a, B, s);
+  LM_CASE(64, 64) LM_CASE(128, 64) LM_CASE(256, 64) LM_CASE(512, 64) LM_CASE(64, 128) LM_CASE(128, 128) LM_CASE(256, 128)
+  LM_CASE(512, 128)
+#undef LM_CASE
+  return LM_EINVAL;
+}

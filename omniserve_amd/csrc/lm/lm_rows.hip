@@ -59,11 +59,13 @@ __device__ __forceinline__ void normalise(f32x4 (&v)[NV], Row<TH>& row, int n, i
 
 struct ResidualArgs {
   float* x; int64_t ldx;                     // residual stream
-  const int* tokens; const elem_t* embed;    // tokens: the residual starts as these rows of the table [vocab][ldx]
+  const int* tokens; const elem_t* embed;    // tokens: the residual starts as these rows of the table [vocab][ldx] ...
+  float embed_scale;                         // ... times this
   const elem_t* y; int64_t ldy;              // sublayer output (or null): added to the residual
+  const float* y_bias;                       // added to y (or null)
   const float* pair_w; int top, pairs0, shared;   // top > 0: y holds expert outputs by (token, choice), see moe_sum
   const float *post_w, *post_b;              // norm of the sublayer output before it is added (or null)
-  const float *next_w, *next_b;              // norm of the new residual for the next sublayer (or null) -> h
+  const float *next_w, *next_b;              // norm of the new residual for the next sublayer (or null: as it is) -> h
   elem_t* h; int64_t ldh;
   const int* rows;                           // row r of the launch works on token rows[r] (or null: r) and writes h[r]
   int n, kind, store_x;
@@ -83,7 +85,7 @@ __global__ __launch_bounds__(TH) void residual_norm_kernel(ResidualArgs p) {
     const int c = 4 * (TH * i + tid);
     x[i] = y[i] = zero4();
     if (c >= p.n) continue;
-    x[i] = er ? from_quad(*(const quad_t*)(er + c)) : *(const f32x4*)(xr + c);
+    x[i] = er ? p.embed_scale * from_quad(*(const quad_t*)(er + c)) : *(const f32x4*)(xr + c);
   }
   if (p.y) {
     if (p.top > 0) {      // weighted sum of the chosen experts' rows (+ the shared expert's)
@@ -117,6 +119,13 @@ __global__ __launch_bounds__(TH) void residual_norm_kernel(ResidualArgs p) {
         if (c < p.n) y[i] += from_quad(*(const quad_t*)(yr + c));
       }
     }
+    if (p.y_bias) {
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int c = 4 * (TH * i + tid);
+        if (c < p.n) y[i] += *(const f32x4*)(p.y_bias + c);
+      }
+    }
     if (p.post_w) normalise<TH, NV>(y, row, p.n, p.kind, p.eps, p.post_w, p.post_b);
 #pragma unroll
     for (int i = 0; i < NV; ++i) x[i] += y[i];
@@ -128,8 +137,8 @@ __global__ __launch_bounds__(TH) void residual_norm_kernel(ResidualArgs p) {
       if (c < p.ldx) *(f32x4*)(xr + c) = x[i];
     }
   }
-  if (!p.next_w) return;
-  normalise<TH, NV>(x, row, p.n, p.kind, p.eps, p.next_w, p.next_b);
+  if (!p.h) return;
+  if (p.next_w) normalise<TH, NV>(x, row, p.n, p.kind, p.eps, p.next_w, p.next_b);
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
     const int c = 4 * (TH * i + tid);
@@ -163,6 +172,41 @@ __global__ __launch_bounds__(ROW_THREADS) void gated_rms_kernel(elem_t* out, int
 #pragma unroll
     for (int e = 0; e < 4; ++e) y[e] = v[i][e] * r * ww[e] * sigmoid(g[e]);
     *(quad_t*)(out + (int64_t)t * ldo + c) = to_quad(y);
+  }
+}
+
+// Per head: out = rms_norm(o over n of dv columns) * w * act(gate).  dv / 4 lanes per head.
+__global__ __launch_bounds__(ROW_THREADS) void gated_head_rms_kernel(elem_t* out, int64_t ldo, const elem_t* o, int64_t ldi,
+                                                                     const elem_t* gate, int64_t ldg, const float* w, int cols, int dv,
+                                                                     int n, float eps, int act) {
+  const int t = blockIdx.x, lanes = dv / 4;
+  for (int c = 4 * (int)threadIdx.x; c < cols; c += 4 * ROW_THREADS) {
+    const f32x4 v = from_quad(*(const quad_t*)(o + (int64_t)t * ldi + c)), g = from_quad(*(const quad_t*)(gate + (int64_t)t * ldg + c));
+    float ss = (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]);      // (padded columns hold zeros)
+    for (int m = lanes >> 1; m > 0; m >>= 1) ss += __shfl_xor(ss, m, 64);
+    const float r = 1.0f / sqrtf(ss / (float)n + eps);
+    const f32x4 ww = *(const f32x4*)(w + c % dv);
+    f32x4 y;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) y[e] = v[e] * r * ww[e] * (act == LM_ACT_SILU ? silu(g[e]) : sigmoid(g[e]));
+    *(quad_t*)(out + (int64_t)t * ldo + c) = to_quad(y);
+  }
+}
+
+// gated unit of rows in alternating blocks of 16 gate and 16 up channels
+__global__ __launch_bounds__(ROW_THREADS) void glu_kernel(elem_t* out, int64_t ldo, const elem_t* x, int64_t ldx, const float* bias, int n,
+                                                          int act) {
+  const int64_t t = blockIdx.x;
+  for (int c = FR * (int)threadIdx.x; c < n; c += FR * ROW_THREADS) {
+    const int s = 32 * (c >> 4) + (c & 15);
+    const frag_t g = *(const frag_t*)(x + t * ldx + s), u = *(const frag_t*)(x + t * ldx + s + 16);
+    frag_t r;
+#pragma unroll
+    for (int e = 0; e < FR; ++e) {
+      const float a = (float)g[e] + (bias ? bias[s + e] : 0.f), b = (float)u[e] + (bias ? bias[s + 16 + e] : 0.f);
+      r[e] = (elem_t)((act == LM_ACT_GELU_TANH ? gelu_tanh(a) : silu(a)) * b);
+    }
+    *(frag_t*)(out + t * ldo + c) = r;
   }
 }
 
@@ -255,14 +299,14 @@ __global__ __launch_bounds__(1024) void argmax_kernel(int64_t* out, const float*
 
 using namespace lm;
 
-extern "C" int lm_residual_norm(float* x, int64_t ldx, const int* tokens, const void* embed, const void* y, int64_t ldy,
-                                const float* pair_w, int top, int pairs0, int shared, const float* post_w, const float* post_b,
+extern "C" int lm_residual_norm(float* x, int64_t ldx, const int* tokens, const void* embed, float embed_scale, const void* y,
+                                int64_t ldy, const float* y_bias, const float* pair_w, int top, int pairs0, int shared, const float* post_w, const float* post_b,
                                 const float* next_w, const float* next_b, void* h, int64_t ldh, const int* rows, int n_rows, int n,
                                 int kind, int store_x, float eps, void* stream) {
-  if (n_rows <= 0 || n <= 0 || n > ldx || ldx % 4 || (tokens && !embed) || (next_w && (!h || ldh % 4 || ldh < n)) || top < 0 ||
+  if (n_rows <= 0 || n <= 0 || n > ldx || ldx % 4 || (tokens && !embed) || (next_w && !h) || (h && (ldh % 4 || ldh < n)) || top < 0 ||
       (top > 0 && (!y || !pair_w)))
     return LM_EINVAL;
-  ResidualArgs a{x, ldx, tokens, (const elem_t*)embed, (const elem_t*)y, ldy, pair_w, top, pairs0, shared, post_w, post_b, next_w,
+  ResidualArgs a{x, ldx, tokens, (const elem_t*)embed, embed_scale, (const elem_t*)y, ldy, y_bias, pair_w, top, pairs0, shared, post_w, post_b, next_w,
                  next_b, (elem_t*)h, ldh, rows, n, kind, store_x, eps};
   hipStream_t s = (hipStream_t)stream;
   const int64_t cols = ldx > ldh ? ldx : ldh;
@@ -290,6 +334,23 @@ extern "C" int lm_gated_rms(void* out, int64_t ldo, const void* o, int64_t ldi, 
   LM_CASE(1) LM_CASE(2) LM_CASE(4) LM_CASE(8) LM_CASE(16)
 #undef LM_CASE
   return LM_EINVAL;
+}
+
+extern "C" int lm_gated_head_rms(void* out, int64_t ldo, const void* o, int64_t ldi, const void* gate, int64_t ldg, const float* w,
+                                 int rows, int H, int dv, int n, float eps, int act, void* stream) {
+  if (rows <= 0 || H <= 0 || (dv != 64 && dv != 128 && dv != 256) || n <= 0 || n > dv || ldo % 4 || ldi % 4 || ldg % 4 ||
+      (act != LM_ACT_SILU && act != LM_ACT_SIGMOID))
+    return LM_EINVAL;
+  hipLaunchKernelGGL(gated_head_rms_kernel, dim3(rows), dim3(ROW_THREADS), 0, (hipStream_t)stream, (elem_t*)out, ldo, (const elem_t*)o,
+                     ldi, (const elem_t*)gate, ldg, w, H * dv, dv, n, eps, act);
+  return launch_status();
+}
+
+extern "C" int lm_glu(void* out, int64_t ldo, const void* x, int64_t ldx, const float* bias, int rows, int n, int act, void* stream) {
+  if (rows <= 0 || n <= 0 || n % 16 || ldo % FR || ldx % FR || (act != LM_ACT_SILU && act != LM_ACT_GELU_TANH)) return LM_EINVAL;
+  hipLaunchKernelGGL(glu_kernel, dim3(rows), dim3(ROW_THREADS), 0, (hipStream_t)stream, (elem_t*)out, ldo, (const elem_t*)x, ldx, bias, n,
+                     act);
+  return launch_status();
 }
 
 extern "C" int lm_rope_append(void* qkv, int64_t ld, const void* v_first, int64_t ldv, float lambda, const float* freq, int half,

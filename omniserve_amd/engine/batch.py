@@ -32,8 +32,13 @@ class DeviceBatch:
     attn_tiles: torch.Tensor  # [., 2] portion, first row
     segments: torch.Tensor    # [., 8]
     block_table: torch.Tensor # [n_entries + n_decode, pages]
+    portions: torch.Tensor = None      # [n_entries, 8] first token, tokens, state slot, starts from zero, first chunk, chunks, position, 0
+    chunks: torch.Tensor = None        # [.] portion of every chunk
+    context_pages: torch.Tensor = None # pages of the portions' contexts, one portion behind the other
+    context_table: torch.Tensor = None # [n_entries, pages] place of a portion's page among those of its expansion
     segment_len: int = 64
     multi_segment: bool = False
+    expansions: tuple = ()             # (first context page, pages, first tile, tiles) of portions whose contexts are expanded at once
 
 
 class BatchBuilder:
@@ -42,6 +47,7 @@ class BatchBuilder:
     def __init__(self, model, device):
         self.page, self.attn_rows, self.device = model.page_size, model.attn_rows, device
         self.linear_wgs = model.linear_workgroups()
+        self.chunk, self.expand = model.chunk_rows, model.expand_pages
 
     def _segment_len(self, portions: List[Entry]) -> int:
         """Tokens per segment of a recurrent layer: enough segments for two workgroups per CU, none below 256 tokens, at most 32
@@ -62,6 +68,8 @@ class BatchBuilder:
         tokens, pos, slot = (np.zeros((T,), np.int32) for _ in range(3))
         table = np.zeros((N, width), np.int32)
         ent, tiles, segs, rows, wanted = [], [], [], [], []
+        ports, chunks, context, groups = [], [], [], []
+        context_table = np.zeros((len(portions) if self.expand else 0, width), np.int32)
         seg_len, multi, at = 64, False, 0
         if portions:
             seg_len = self._segment_len(portions)
@@ -76,7 +84,19 @@ class BatchBuilder:
                 table[k, :e.seq.pages] = np.maximum(e.seq.table[:e.seq.pages], 0)
             if n > 1:
                 ent.append((at, n, p0, k))
-                tiles += [(k, r) for r in range(0, n, self.attn_rows)]
+                here = [(k, r) for r in range(0, n, self.attn_rows)]
+                if self.expand:
+                    if not groups or groups[-1][1] + e.seq.pages > self.expand:
+                        groups.append([len(context), 0, len(tiles), 0])
+                    context_table[k, :e.seq.pages] = groups[-1][1] + np.arange(e.seq.pages)
+                    context += table[k, :e.seq.pages].tolist()
+                    groups[-1][1] += e.seq.pages
+                    groups[-1][3] += len(here)
+                tiles += here
+                if self.chunk:
+                    nc = -(-n // self.chunk)
+                    ports.append((at, n, e.seq.slot, int(p0 == 0), len(chunks), nc, p0, 0))
+                    chunks += [len(ports) - 1] * nc
                 ns = -(-n // seg_len)
                 multi |= ns > 1
                 segs += [(at + s * seg_len, min(seg_len, n - s * seg_len), e.seq.slot, int(p0 == 0), s, ns, 0, 0) for s in range(ns)]
@@ -86,10 +106,12 @@ class BatchBuilder:
             at += n
         parts = [tokens, pos, slot, np.array([e.seq.slot for e in single], np.int32), np.array(rows, np.int32),
                  np.array(ent, np.int32).reshape(-1, 4), np.array(tiles, np.int32).reshape(-1, 2),
-                 np.array(segs, np.int32).reshape(-1, 8), table]
+                 np.array(segs, np.int32).reshape(-1, 8), table, np.array(ports, np.int32).reshape(-1, 8), np.array(chunks, np.int32),
+                 np.array(context, np.int32), context_table]
         d = self._upload(parts)
         longest = max(e.seq.length + len(e.tokens) for e in entries)
-        return DeviceBatch(n_prompt, n_decode, len(portions), longest, *d, segment_len=seg_len, multi_segment=multi), wanted
+        return DeviceBatch(n_prompt, n_decode, len(portions), longest, *d, segment_len=seg_len, multi_segment=multi,
+                           expansions=tuple(map(tuple, groups))), wanted
 
     def _upload(self, parts):
         sizes = [p.size for p in parts]

@@ -2,7 +2,7 @@
 layer's state.
 
 One page number stands for 64 tokens in every attention layer (each layer has its own K and V pool, [pages][kv heads][64][size]);
-one slot number for a sequence's state in every recurrent layer ([slots][heads][dk][dv], f32).  A slot needs no clearing: a
+one slot number for a sequence's state in every recurrent layer ([slots][heads][dk][dv] and rings of convolution inputs, f32).  A slot needs no clearing: a
 sequence's first step starts its state from zero."""
 from __future__ import annotations
 
@@ -41,7 +41,7 @@ class Cache:
         if not self.paged:
             num_pages = 0
         self.kv = model.page_pools(num_pages, device)
-        self.state = [torch.zeros((num_slots, h, dk, dv), dtype=torch.float32, device=device) for h, dk, dv in model.state_shapes()]
+        self.state = [torch.zeros((num_slots, *shape), dtype=torch.float32, device=device) for shape in model.state_shapes()]
         self._pages: List[int] = list(range(num_pages))[::-1]
         self._slots: List[int] = list(range(num_slots))[::-1]
 

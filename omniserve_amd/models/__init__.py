@@ -8,6 +8,7 @@ import os
 
 # architecture name -> (module, class)
 _REGISTRY = {
+    "Bagedra": ("omniserve_amd.models.bagedra", "Bagedra"),
     "Bobavik": ("omniserve_amd.models.bobavik", "Bobavik"),
     "LlamaForCausalLM": ("omniserve_amd.models.qserve_llama", "QServeLlama"),
 }

@@ -11,6 +11,8 @@ class EngineModel:
 
     page_size = 64                       # tokens per cache page
     attn_rows = 128                      # query rows of one prefill attention tile
+    chunk_rows = 0                       # tokens per chunk of recurrent layers that work in chunks (0: there are none)
+    expand_pages = 0                     # most context pages a layer expands into keys and values at once (0: none does)
     dtypes: Tuple[torch.dtype, ...] = () # number formats the model runs in, its default first
     capturable = True                    # single-token steps may be captured in HIP graphs (empty places: position < 0)
     vocab: int
@@ -28,11 +30,12 @@ class EngineModel:
 
     # ---- what the cache holds for a sequence ----
     def kv_shapes(self) -> List[Tuple[int, int, int]]:
-        """(kv heads, key size, value size) of every layer that keeps keys and values"""
+        """(kv heads, key size, value size) of every layer that keeps keys and values (a latent row: 1, its size, 0)"""
         return []
 
-    def state_shapes(self) -> List[Tuple[int, int, int]]:
-        """(heads, key size, value size) of every recurrent layer's f32 state"""
+    def state_shapes(self) -> List[Tuple[int, ...]]:
+        """One sequence's part of every f32 tensor that recurrent layers keep: a state (heads, key size, value size), a ring of a
+        convolution's inputs (rows, channels)"""
         return []
 
     def page_pools(self, num_pages: int, device):

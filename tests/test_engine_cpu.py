@@ -198,8 +198,8 @@ def test_registry_and_config():
     assert (spec.width, spec.vocab, spec.eps, spec.logit_scale, spec.norm) == (72, 33, 1e-3, 0.7, "layer")
     a, b, c = (l.mixer for l in spec.layers)
     assert (a.window, a.rotary.dims, a.rotary.base, a.value_mix, a.rotary.scaling["factor"]) == (9, 16, 777.0, True, 8.0)
-    assert b.decay == (0.55, 0.93, 0.9985) and spec.layers[1].moe is None
-    assert not c.value_mix and c.rotary.scaling is None and spec.layers[2].moe == layers.MoeSpec(6, 1, 48, None)
+    assert b.decay == (0.55, 0.93, 0.9985) and spec.layers[1].ff is None
+    assert not c.value_mix and c.rotary.scaling is None and spec.layers[2].ff == layers.MoeSpec(6, 1, 48, None)
     for bad in (dict(attention(), type="other"), dict(attention(), mlp={"kind": "dense"}), lightning(decay=[0.5, 1.5, 0.1]), lightning(decay=[0.5, 0.2]),
                 attention(heads=3, kv_heads=2), attention(scale=-1.0), attention(window=0), attention(rot=50)):
         with pytest.raises(ValueError):

@@ -39,7 +39,7 @@ class OneMixer(EngineModel):
         return [self.mixer.cache_shape()] if self.soft else []
 
     def state_shapes(self):
-        return [] if self.soft else [self.mixer.state_shape()]
+        return [] if self.soft else self.mixer.state_shapes()
 
     def window(self):
         return self.layer["mixer"]["mask"]["size"] if self.soft else 1
@@ -213,9 +213,9 @@ def test_mixture(kind, tokens, dtype):
     x = torch.zeros((tokens, W), dtype=dtype, device=DEV)
     x[:, :width] = torch.from_numpy(h).to(DEV, dtype)
     y, experts = mix(x)
-    assert np.abs(experts[0].cpu().numpy() - wt).max() < 1e-4
+    assert np.abs(experts["experts"][0].cpu().numpy() - wt).max() < 1e-4
     r = torch.zeros((tokens, W), dtype=F32, device=DEV)
-    ops.residual_norm(r, width, "layer", 1e-5, y=y, experts=experts)          # the weighted sum alone
+    ops.residual_norm(r, width, "layer", 1e-5, y=y, **experts)                # the weighted sum alone
     e = errors(r[:, :width].cpu().numpy(), want)
     assert e.max() < TOL[dtype], e.max()
 
