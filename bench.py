@@ -678,10 +678,16 @@ def design_bench(args):
     from omniserve_amd.engine import benchmark
     device = torch.device("cuda:0")
     torch.cuda.set_device(device)
-    sizes = tuple(benchmark.SIZES) if args.design == "all" else (args.design,)
-    res = benchmark.run(device, sizes, llama=not args.no_extras)
-    first = res[sizes[0]]["bobavik_bf16"]["decode_bs16"]
-    print(json.dumps({"metric": "decode tokens/s, Bobavik %s, bs 16, 1024 cached tokens" % sizes[0], "value": first["tokens_per_s"],
+    table = benchmark.BAGEDRA_SIZES if args.architecture == "Bagedra" else benchmark.SIZES
+    sizes = tuple(table) if args.design == "all" else (args.design,)
+    if not set(sizes) <= set(table):
+        raise SystemExit("--design: unknown size (known: %s)" % ", ".join(table))
+    if args.architecture == "Bagedra":
+        res = benchmark.run_bagedra(device, sizes, beside=not args.no_extras)
+    else:
+        res = benchmark.run(device, sizes, llama=not args.no_extras)
+    first = res[sizes[0]][args.architecture.lower() + "_bf16"]["decode_bs16"]
+    print(json.dumps({"metric": "decode tokens/s, %s %s, bs 16, 1024 cached tokens" % (args.architecture, sizes[0]), "value": first["tokens_per_s"],
                       "unit": "tokens/s", "n_gpus": 1, "ms_per_step": first["ms_per_step"], "higher_is_better": True,
                       "vs_baseline": None, "dtype": "bf16", "data": "synthetic (random weights and tokens)", "designs": res}), flush=True)
 
@@ -714,6 +720,8 @@ def main():
     ap.add_argument("--design", nargs="?", const="all", default=None, metavar="SIZE",
                     help="instead of the workload above: prefill and decode throughput of the Bobavik design at real layer sizes beside "
                          "the W4A8KV4 Llama of equal size (omniserve_amd/engine/benchmark.py; SIZE: all, 4096 or 2048)")
+    ap.add_argument("--architecture", choices=["Bobavik", "Bagedra"], default="Bobavik",
+                    help="with --design: Bagedra runs beside a Bobavik of its width, heads and feed-forward")
     args = ap.parse_args()
     if args.design:
         return design_bench(args)

@@ -109,12 +109,13 @@ int lm_gla_decode(const void* x, int64_t ld, void* o, int64_t ldo, float* state,
  * last row: the current input) and silu; q and k become unit vectors (eps qk_eps), q times scale.  ring: f32 [slots][taps][channels],
  * the input of position p in row p % taps.
  * portion [.][8]: first token, tokens, slot, starts from zero, first chunk, chunks, position, 0; chunks [n_chunks]: portion of every
- * chunk of lm_delta_chunk_rows() tokens.  y: the convolved rows [tokens][channels], norms: f32 [tokens][2 G], mats: elem
+ * chunk of lm_delta_chunk_rows() tokens.  seg, multi as in lm_linear_prefill, every segment of whole chunks but a portion's last, its
+ * first chunk in column 6; seg_state: f32 [segments][H][dk * (dv + dk)].  y: the convolved rows [tokens][channels], norms: f32 [tokens][2 G], mats: elem
  * [n_chunks][H][2][operands][rows][rows], vecs: f32 [n_chunks][H][4][rows]. */
 int lm_delta_chunk_rows(void);
 int64_t lm_delta_mat_elems(void);
-int lm_delta_prefill(const void* x, int64_t ld, void* o, int64_t ldo, float* state, float* ring, const int* portion, int portions,
-                     const int* chunks, int n_chunks, const float* conv_w, int taps, float qk_eps, float scale, int64_t ab_col,
+int lm_delta_prefill(const void* x, int64_t ld, void* o, int64_t ldo, float* state, float* ring, float* seg_state, const int* portion,
+                     const int* chunks, int n_chunks, const int* seg, int segments, int multi, const float* conv_w, int taps, float qk_eps, float scale, int64_t ab_col,
                      const float* a_log, const float* dt_bias, void* y, float* norms, void* mats, float* vecs, int H, int G, int dk,
                      int dv, void* stream);
 int lm_delta_decode(const void* x, int64_t ld, void* o, int64_t ldo, float* state, float* ring, const int* slot, const int* pos,

@@ -53,8 +53,8 @@ PROTOTYPES = {
     "lm_gla_decode": (_i, [_vp, _i64, _vp, _i64, _vp, _vp, _vp, _i64, _vp, _vp, _i, _f, _f, _i64, _vp, _i, _f, _i, _i, _i, _i, _vp]),
     "lm_delta_chunk_rows": (_i, []),
     "lm_delta_mat_elems": (_i64, []),
-    "lm_delta_prefill": (_i, [_vp, _i64, _vp, _i64, _vp, _vp, _vp, _i, _vp, _i, _vp, _i, _f, _f, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i,
-                              _i, _i, _vp]),
+    "lm_delta_prefill": (_i, [_vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _vp, _i, _vp, _i, _i, _vp, _i, _f, _f, _i64, _vp, _vp, _vp, _vp,
+                              _vp, _vp, _i, _i, _i, _i, _vp]),
     "lm_delta_decode": (_i, [_vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _vp, _i, _f, _f, _i64, _vp, _vp, _i64, _vp, _i, _f, _i, _i, _i, _i,
                              _i, _vp]),
     "lm_route_scratch_words": (_i64, [_i, _i, _i]),
@@ -159,14 +159,15 @@ class LmOps:
         self._call("lm_gla_decode", _p(x), _ld(x), _p(o), _ld(o), _p(state), _p(slot), _p(pos), low_col, _p(a2), _p(bias), a2.shape[1],
                    1.0 / tau, scale, gate_col, _p(w), n, eps, x.shape[0], heads, dk, dv)
 
-    def delta_prefill(self, x, o, state, ring, portions, chunks, conv_w, qk_eps, scale, ab_col, a_log, dt_bias, heads, kv_heads, dk, dv):
+    def delta_prefill(self, x, o, state, ring, portions, chunks, seg, multi, conv_w, qk_eps, scale, ab_col, a_log, dt_bias, heads, kv_heads, dk, dv):
         T, n, dev = x.shape[0], chunks.numel(), x.device
         f32 = lambda *s: torch.empty(s, dtype=torch.float32, device=dev)      # noqa: E731
         y = torch.empty((T, conv_w.shape[1]), dtype=self.dtype, device=dev)
         mats = torch.empty((n * heads * self._h.lm_delta_mat_elems(),), dtype=self.dtype, device=dev)
         norms, vecs = f32(T, 2 * kv_heads), f32(n, heads, 4, self.delta_chunk)
-        self._call("lm_delta_prefill", _p(x), _ld(x), _p(o), _ld(o), _p(state), _p(ring), _p(portions), portions.shape[0], _p(chunks), n,
-                   _p(conv_w), conv_w.shape[0], qk_eps, scale, ab_col, _p(a_log), _p(dt_bias), _p(y), _p(norms), _p(mats), _p(vecs), heads,
+        seg_state = f32(seg.shape[0], heads, dk * (dv + dk)) if multi else None
+        self._call("lm_delta_prefill", _p(x), _ld(x), _p(o), _ld(o), _p(state), _p(ring), _p(seg_state), _p(portions), _p(chunks), n, _p(seg),
+                   seg.shape[0], int(multi), _p(conv_w), conv_w.shape[0], qk_eps, scale, ab_col, _p(a_log), _p(dt_bias), _p(y), _p(norms), _p(mats), _p(vecs), heads,
                    kv_heads, dk, dv)
 
     def delta_decode(self, x, o, state, ring, slot, pos, conv_w, qk_eps, scale, ab_col, a_log, dt_bias, gate_col, w, n, eps, heads, kv_heads,

@@ -119,6 +119,32 @@ template <int ROWB>
 struct Tile {
   static constexpr int NS = ROWB / 16;
   static_assert(NS >= 8 && NS % 8 == 0, "row size");
+  // The same accesses from per-lane byte offsets, for rows of a power of two bytes: what depends on the block is one XOR.  A loop
+  // that keeps the three offsets from the optimiser (Offsets::forget) does not hold an address register per block.
+  struct Offsets {
+    int frag, quad, col;
+    __device__ __forceinline__ Offsets(int l15, int l4) {
+      static_assert((NS & (NS - 1)) == 0, "row size");
+      const int row = l15 * ROWB, r = 4 * l4 + (l15 >> 2);
+      frag = row + ((l4 ^ swizzle(l15)) << 4);
+      quad = sizeof(elem_t) == 2 ? row + (((l4 >> 1) ^ swizzle(l15)) << 4) + 8 * (l4 & 1) : frag;
+      col = r * ROWB + ((((l15 & 3) >> 1) ^ swizzle(r)) << 4) + 8 * (l15 & 1);
+    }
+    __device__ __forceinline__ void forget() { asm volatile("" : "+v"(frag), "+v"(quad), "+v"(col)); }
+  };
+  __device__ __forceinline__ static frag_t frag(const uint8_t* t, const Offsets& o, int row0, int k) {      // row row0 + l15, step k
+    return *(const frag_t*)(t + row0 * ROWB + (o.frag ^ (k << 6)));
+  }
+  __device__ __forceinline__ static quad_t quad(const uint8_t* t, const Offsets& o, int row0, int blk) {
+    return *(const quad_t*)(t + row0 * ROWB + (o.quad ^ (blk * 16 * (int)sizeof(elem_t))));
+  }
+  __device__ __forceinline__ static quad_t column_quad(const uint8_t* t, const Offsets& o, int row0, int cblk, int l15, int l4) {
+#if LM_ELEM == 0
+    return transposed(t + row0 * ROWB + (o.col ^ (cblk << 5)));
+#else
+    return column_quad(t, row0, cblk, l15, l4);
+#endif
+  }
   __device__ __forceinline__ static int swizzle(int row) {
     if constexpr (NS / 8 % 2 == 1) { // an odd number of half lines: neighbouring rows start in different halves
       const int q = (row >> 1) & 7;
@@ -138,15 +164,19 @@ struct Tile {
   __device__ __forceinline__ static quad_t quad(const uint8_t* t, int row, int blk, int l4) {
     return *(const quad_t*)(t + at(row, 16 * blk + 4 * l4));
   }
-  // column 16 cblk + l15 of rows row0 + 4 l4 + (0..3)
-  __device__ __forceinline__ static quad_t column_quad(const uint8_t* t, int row0, int cblk, int l15, int l4) {
 #if LM_ELEM == 0
-    // lane L of a 16-lane group passes the address of elements 4 (L & 3) .. + 3 of row L >> 2 and receives column L
-    const uint8_t* p = t + at(row0 + 4 * l4 + (l15 >> 2), 16 * cblk + 4 * (l15 & 3));
+  __device__ __forceinline__ static quad_t transposed(const uint8_t* p) {
     typedef __bf16 tr4 __attribute__((__vector_size__(4 * sizeof(__bf16))));
     const tr4 r = __builtin_amdgcn_ds_read_tr16_b64_v4bf16(
         (__attribute__((address_space(3))) tr4*)(__attribute__((address_space(3))) void*)(p));
     return (quad_t){r[0], r[1], r[2], r[3]};
+  }
+#endif
+  // column 16 cblk + l15 of rows row0 + 4 l4 + (0..3)
+  __device__ __forceinline__ static quad_t column_quad(const uint8_t* t, int row0, int cblk, int l15, int l4) {
+#if LM_ELEM == 0
+    // lane L of a 16-lane group passes the address of elements 4 (L & 3) .. + 3 of row L >> 2 and receives column L
+    return transposed(t + at(row0 + 4 * l4 + (l15 >> 2), 16 * cblk + 4 * (l15 & 3)));
 #else
     quad_t q;
 #pragma unroll

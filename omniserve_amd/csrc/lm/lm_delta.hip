@@ -10,8 +10,11 @@
 //   conv      convolution + silu of every channel, the factors rq and rk (parallel over tokens)
 //   chunk     one wave per (chunk, head): A and P by MFMA, T = (I + A)^-1 diag(beta) by forward substitution, one column per lane;
 //             the last inputs of a portion go to the ring of its slot
-//   prefill   one workgroup per (portion, head, 64 value columns) walks the chunks: R = V - diag(e^G rk) K~ S, U = T R, the outputs
+//   prefill   one workgroup per (segment, head, 64 value columns) walks the chunks: R = V - diag(e^G rk) K~ S, U = T R, the outputs
 //             and the next state.  S stays in MFMA accumulators; every result tile is the next product's operand as it lies.
+// Long portions are cut into segments that run in parallel.  A segment takes a state S to M S + C: a first pass forms C (the segment
+// from a zero state) and, as dk more columns, M (the segment without values, from the identity); the second pass starts every segment
+// from the states these give.
 // f32 factors (S, R, U, T, P) enter the bf16 products as two bf16 operands each; of two such factors the product of the two low
 // parts is dropped.
 #include "lm_state.h"
@@ -29,6 +32,9 @@ struct DeltaArgs {
   float* ring;                           // [slots][taps][channels]: the input of position p in row p % taps
   const int* portion;                    // [.][8]: first token, tokens, slot, 1 = starts from zero, first chunk, chunks, position, 0
   const int* chunks;                     // [n_chunks]: its portion
+  const int* seg;                        // [segments][8]: first token, tokens, slot, 1 = starts from zero, index in its portion,
+                                         //                segments of the portion, first chunk, 0
+  float* seg_state;                      // [segments][H]: C [dk * dv] as the accumulators hold it, M [dk][dk]
   const float* conv_w; int taps;         // [taps][channels], the last row meets the current token
   float qk_eps, scale;
   int64_t ab_col;
@@ -41,8 +47,10 @@ struct DeltaArgs {
 };
 
 // ---- convolution, silu, unit-vector factors; 256 threads x FR channels, CONV_TOKENS tokens of a chunk ----
-constexpr int CONV_TOKENS = 8;
+constexpr int CONV_TOKENS = 16;
 
+// TAPS > 0: taps known, weights and the inputs on their way through stay in registers; 0: any number
+template <int TAPS>
 __global__ __launch_bounds__(256) void delta_conv_kernel(DeltaArgs p) {
   const int channels = 2 * p.G * p.dk + p.H * p.dv, c = (blockIdx.y * 256 + threadIdx.x) * FR;
   const int ck = blockIdx.x / (DC / CONV_TOKENS), part = blockIdx.x % (DC / CONV_TOKENS);
@@ -51,23 +59,17 @@ __global__ __launch_bounds__(256) void delta_conv_kernel(DeltaArgs p) {
   const int t0 = (ck - pp[4]) * DC + part * CONV_TOKENS;       // within the portion
   if (c >= channels) return;
   const int qk = p.G * p.dk, lanes = p.dk / FR;
-  for (int t = t0; t < min(t0 + CONV_TOKENS, count); ++t) {
-    float s[FR];
+  auto input = [&](int t) -> frag_t {                           // of place t, which may lie before the portion
+    if (t >= 0) return *(const frag_t*)(p.x + (int64_t)(first + t) * p.ld + c);
+    frag_t v = {};
+    if (pos0 + t >= 0) {
+      const float* r = p.ring + ((int64_t)slot * p.taps + (pos0 + t) % p.taps) * channels + c;
 #pragma unroll
-    for (int e = 0; e < FR; ++e) s[e] = 0.f;
-    for (int j = 0; j < p.taps; ++j) {                          // input t - j
-      const float* w = p.conv_w + (int64_t)(p.taps - 1 - j) * channels + c;
-      const int back = t - j;
-      if (back >= 0) {
-        const frag_t v = *(const frag_t*)(p.x + (int64_t)(first + back) * p.ld + c);
-#pragma unroll
-        for (int e = 0; e < FR; ++e) s[e] += w[e] * (float)v[e];
-      } else if (pos0 + back >= 0) {
-        const float* v = p.ring + ((int64_t)slot * p.taps + (pos0 + back) % p.taps) * channels + c;
-#pragma unroll
-        for (int e = 0; e < FR; ++e) s[e] += w[e] * v[e];
-      }
+      for (int e = 0; e < FR; ++e) v[e] = (elem_t)r[e];         // (an element's value)
     }
+    return v;
+  };
+  auto finish = [&](int t, const float (&s)[FR]) {
     frag_t y;
     float ss = 0.f;
 #pragma unroll
@@ -80,6 +82,49 @@ __global__ __launch_bounds__(256) void delta_conv_kernel(DeltaArgs p) {
       for (int m = lanes >> 1; m > 0; m >>= 1) ss += __shfl_xor(ss, m, 64);
       if (c % p.dk == 0)
         p.norms[(int64_t)(first + t) * 2 * p.G + c / p.dk] = (c < qk ? p.scale : 1.0f) / sqrtf(ss + p.qk_eps);
+    }
+  };
+  const int t1 = min(t0 + CONV_TOKENS, count);
+  if constexpr (TAPS > 0) {
+    if (t0 >= t1) return;
+    constexpr int B = 4;                                        // inputs requested together
+    float w[TAPS][FR];
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+      for (int e = 0; e < FR; ++e) w[j][e] = p.conv_w[(int64_t)j * channels + c + e];
+    frag_t in[TAPS - 1 + B];
+#pragma unroll
+    for (int j = 0; j < TAPS - 1; ++j) in[j] = input(t0 - (TAPS - 1) + j);
+    for (int t = t0; t < t1; t += B) {
+#pragma unroll
+      for (int b = 0; b < B; ++b) in[TAPS - 1 + b] = input(min(t + b, t1 - 1));
+#pragma unroll
+      for (int b = 0; b < B; ++b) {
+        if (t + b >= t1) break;
+        float s[FR];
+#pragma unroll
+        for (int e = 0; e < FR; ++e) s[e] = 0.f;
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+          for (int e = 0; e < FR; ++e) s[e] += w[j][e] * (float)in[b + j][e];
+        finish(t + b, s);
+      }
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) in[j] = in[B + j];
+    }
+  } else {
+    for (int t = t0; t < t1; ++t) {
+      float s[FR];
+#pragma unroll
+      for (int e = 0; e < FR; ++e) s[e] = 0.f;
+      for (int j = 0; j < p.taps; ++j) {
+        const frag_t v = input(t - (p.taps - 1) + j);
+#pragma unroll
+        for (int e = 0; e < FR; ++e) s[e] += p.conv_w[(int64_t)j * channels + c + e] * (float)v[e];
+      }
+      finish(t, s);
     }
   }
 }
@@ -209,8 +254,8 @@ struct DeltaGeom {
   static_assert(NQ >= 1 && NV >= 1 && NM >= 1 && 2 * NOPND * DC * MR % TH == 0, "loads");
 };
 
-template <int DK>
-__global__ __launch_bounds__(256, 1) void delta_prefill_kernel(DeltaArgs p) {
+template <int DK, bool OUTPUT>
+__global__ __launch_bounds__(256, SPLIT && DK <= 128 ? 2 : 1) void delta_prefill_kernel(DeltaArgs p) {
   typedef DeltaGeom<DK> Gm;
   typedef Tile<Gm::KB> KT;
   typedef Tile<Gm::VB> VT;
@@ -219,50 +264,110 @@ __global__ __launch_bounds__(256, 1) void delta_prefill_kernel(DeltaArgs p) {
   uint8_t *qt = lds + Gm::Q0, *kt = lds + Gm::K0, *vt = lds + Gm::V0, *mt = lds + Gm::M0;
   float* vec = (float*)(lds + Gm::S0);
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l15 = lane & 15, l4 = lane >> 4;
-  const int* pp = p.portion + 8 * blockIdx.x;
-  const int row0 = pp[0], count = pp[1], slot = pp[2], fresh = pp[3], ck0 = pp[4], nch = pp[5];
-  const int h = blockIdx.y, g = h / (p.H / p.G), dv0 = Gm::DVB * blockIdx.z;
+  const int sg = blockIdx.x;
+  const int* sp = p.seg + 8 * sg;
+  const int row0 = sp[0], count = sp[1], slot = sp[2], fresh = sp[3], idx = sp[4], nseg = sp[5], ck0 = sp[6], nch = (count + DC - 1) / DC;
+  const int h = blockIdx.y, g = h / (p.H / p.G);
+  const bool matrix = !OUTPUT && (int)blockIdx.z >= p.dv / Gm::DVB;      // columns of M
+  const int dv0 = Gm::DVB * (matrix ? blockIdx.z - p.dv / Gm::DVB : blockIdx.z);
+  if (!OUTPUT && (idx == nseg - 1 || (matrix && idx == 0))) return;      // nothing follows; nothing is in front
   const int channels = 2 * p.G * DK + p.H * p.dv;
-  float* own = p.state + ((int64_t)slot * p.H + h) * DK * p.dv + (int64_t)4 * l4 * p.dv + dv0 + 16 * wave + l15;
+  float* own = p.state + ((int64_t)slot * p.H + h) * DK * p.dv;
+  const uint32_t sbase = 4 * l4 * p.dv + dv0 + 16 * wave + l15;         // this lane's column, row 4 l4
   f32x4 S[NS];
 #pragma unroll
-  for (int t = 0; t < NS; ++t)
+  for (int t = 0; t < NS; ++t) S[t] = zero4();
+  auto seg_at = [&](int i) { return p.seg_state + ((int64_t)(sg - idx + i) * p.H + h) * DK * (p.dv + DK); };
+  auto seg_cols = [&](int i) { return (f32x4*)(seg_at(i) + (dv0 + 16 * wave) * DK) + lane; };      // C, this wave's columns
+  auto keep = [&](int i) {
+    f32x4* s = seg_cols(i);
 #pragma unroll
-    for (int r = 0; r < 4; ++r) S[t][r] = fresh ? 0.f : own[(int64_t)(16 * t + r) * p.dv];
+    for (int t = 0; t < NS; ++t) s[64 * t] = S[t];
+  };
+  auto recall = [&](int i) {
+    const f32x4* s = seg_cols(i);
+#pragma unroll
+    for (int t = 0; t < NS; ++t) S[t] = s[64 * t];
+  };
+  if (matrix) {
+#pragma unroll
+    for (int t = 0; t < NS; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) S[t][r] = 16 * t + 4 * l4 + r == dv0 + 16 * wave + l15 ? 1.0f : 0.0f;
+  } else if (idx == 0) {
+    if (OUTPUT && nseg > 1) {
+      recall(nseg - 1);                   // kept by the first pass: the last segment replaces the slot's state
+    } else if (!fresh) {
+#pragma unroll
+      for (int t = 0; t < NS; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) S[t][r] = own[sbase + (uint32_t)((16 * t + r) * p.dv)];
+    }
+    if (!OUTPUT) keep(nseg - 1);
+  } else if (OUTPUT) {
+    recall(0);
+    for (int i = 1; i < idx; ++i) {       // S <- M_i S + C_i
+      const float* m = seg_at(i) + DK * p.dv;
+      const f32x4* c = seg_cols(i);
+      f32x4 N[NS];
+#pragma unroll
+      for (int t = 0; t < NS; ++t) N[t] = c[64 * t];
+#pragma unroll
+      for (int k = 0; k < NS; k += 2) {
+        quad_t s0[NOPND], s1[NOPND];
+        split_quad(S[k], s0);
+        split_quad(S[k + 1], s1);
+#pragma unroll
+        for (int t = 0; t < NS; ++t) {
+          const float* row = m + (uint32_t)((16 * t + l15) * DK + 16 * k + 4 * l4);
+          quad_t a0[NOPND], a1[NOPND];
+          split_quad(*(const f32x4*)row, a0);
+          split_quad(*(const f32x4*)(row + 16), a1);
+#pragma unroll
+          for (int o = 0; o < NOPND; ++o) N[t] = mma_quads(a0[0], a1[0], s0[o], s1[o], N[t]);
+          if constexpr (SPLIT) N[t] = mma_quads(a0[1], a1[1], s0[0], s1[0], N[t]);
+        }
+      }
+#pragma unroll
+      for (int t = 0; t < NS; ++t) S[t] = N[t];
+    }
+  }
 
   const elem_t* src = p.y + (int64_t)row0 * channels;
   const int qo = g * DK, ko = (p.G + g) * DK, vo = 2 * p.G * DK + h * p.dv + dv0;
-  frag_t rq[Gm::NQ], rk[Gm::NQ], rv[Gm::NV], rm[Gm::NM];
+  constexpr int NM = OUTPUT ? Gm::NM : Gm::NM / 2;      // (T comes first)
+  frag_t rq[OUTPUT ? Gm::NQ : 1], rk[Gm::NQ], rv[Gm::NV], rm[NM];
   float rvec = 0.f;
-  auto fetch = [&](int ck) {
-    const int c0 = ck * DC;
+  auto fetch = [&](int ck) {              // addresses: a base all lanes share, 32-bit offsets
+    const elem_t* base = src + (int64_t)ck * DC * channels;
+    const int last = count - 1 - ck * DC;
 #pragma unroll
     for (int i = 0; i < Gm::NQ; ++i) {
       const int sl = Gm::TH * i + tid, r = sl / KT::NS, s = sl % KT::NS;
-      const bool in = c0 + r < count;
-      const elem_t* a = src + (int64_t)(in ? c0 + r : 0) * channels + s * FR;
-      rq[i] = in ? *(const frag_t*)(a + qo) : frag_t{};
-      rk[i] = in ? *(const frag_t*)(a + ko) : frag_t{};
+      const uint32_t off = min(r, last) * channels + s * FR;
+      if constexpr (OUTPUT) rq[i] = *(const frag_t*)(base + qo + off);
+      rk[i] = *(const frag_t*)(base + ko + off);
     }
 #pragma unroll
     for (int i = 0; i < Gm::NV; ++i) {
       const int sl = Gm::TH * i + tid, r = sl / VT::NS, s = sl % VT::NS;
-      const bool in = c0 + r < count;
-      rv[i] = in ? *(const frag_t*)(src + (int64_t)(in ? c0 + r : 0) * channels + vo + s * FR) : frag_t{};
+      rv[i] = matrix ? frag_t{} : *(const frag_t*)(base + vo + (uint32_t)(min(r, last) * channels + s * FR));
     }
-    const int64_t at = (int64_t)(ck0 + ck) * p.H + h;
+    const int64_t block = (int64_t)(ck0 + ck) * p.H + h;
 #pragma unroll
-    for (int i = 0; i < Gm::NM; ++i) rm[i] = *(const frag_t*)(p.mats + at * MATS + (Gm::TH * i + tid) * FR);
-    if (tid < 4 * DC) rvec = p.vecs[at * 4 * DC + tid];
+    for (int i = 0; i < NM; ++i) rm[i] = *(const frag_t*)(p.mats + block * MATS + (uint32_t)((Gm::TH * i + tid) * FR));
+    if (tid < 4 * DC) rvec = (p.vecs + block * 4 * DC)[(uint32_t)tid];
   };
   static_assert(4 * DC <= Gm::TH, "one factor per thread");
   fetch(0);
+  typename KT::Offsets at(l15, l4);
   for (int ck = 0; ck < nch; ++ck) {
     const int n = min(DC, count - ck * DC);
+    at.forget();
 #pragma unroll
     for (int i = 0; i < Gm::NQ; ++i) {
       const int sl = Gm::TH * i + tid, off = KT::slot(sl / KT::NS, sl % KT::NS);
-      *(frag_t*)(qt + off) = rq[i];
+      if constexpr (OUTPUT) *(frag_t*)(qt + off) = rq[i];
       *(frag_t*)(kt + off) = rk[i];
     }
 #pragma unroll
@@ -271,7 +376,7 @@ __global__ __launch_bounds__(256, 1) void delta_prefill_kernel(DeltaArgs p) {
       *(frag_t*)(vt + VT::slot(sl / VT::NS, sl % VT::NS)) = rv[i];
     }
 #pragma unroll
-    for (int i = 0; i < Gm::NM; ++i) {
+    for (int i = 0; i < NM; ++i) {
       const int sl = Gm::TH * i + tid;
       *(frag_t*)(mt + (sl / Gm::MR) * Gm::PB + (sl % Gm::MR) * 16) = rm[i];
     }
@@ -289,12 +394,13 @@ __global__ __launch_bounds__(256, 1) void delta_prefill_kernel(DeltaArgs p) {
       split_quad(S[t + 1], s1);
 #pragma unroll
       for (int u = 0; u < RT; ++u) {
-        const quad_t k0 = KT::quad(kt, 16 * u + l15, t, l4), k1 = KT::quad(kt, 16 * u + l15, t + 1, l4);
-        const quad_t q0 = KT::quad(qt, 16 * u + l15, t, l4), q1 = KT::quad(qt, 16 * u + l15, t + 1, l4);
+        const quad_t k0 = KT::quad(kt, at, 16 * u, t), k1 = KT::quad(kt, at, 16 * u, t + 1);
 #pragma unroll
-        for (int o = 0; o < NOPND; ++o) {
-          R[u] = mma_quads(k0, k1, s0[o], s1[o], R[u]);
-          out[u] = mma_quads(s0[o], s1[o], q0, q1, out[u]);
+        for (int o = 0; o < NOPND; ++o) R[u] = mma_quads(k0, k1, s0[o], s1[o], R[u]);
+        if constexpr (OUTPUT) {
+          const quad_t q0 = KT::quad(qt, at, 16 * u, t), q1 = KT::quad(qt, at, 16 * u, t + 1);
+#pragma unroll
+          for (int o = 0; o < NOPND; ++o) out[u] = mma_quads(s0[o], s1[o], q0, q1, out[u]);
         }
       }
     }
@@ -325,10 +431,12 @@ __global__ __launch_bounds__(256, 1) void delta_prefill_kernel(DeltaArgs p) {
     }
     // O^T += U^T P^T
     quad_t us[RT][NOPND];
+    if constexpr (OUTPUT) {
 #pragma unroll
-    for (int u = 0; u < RT; ++u) split_quad(U[u], us[u]);
+      for (int u = 0; u < RT; ++u) split_quad(U[u], us[u]);
+    }
 #pragma unroll
-    for (int it = 0; it < RT; ++it) {
+    for (int it = 0; it < (OUTPUT ? RT : 0); ++it) {
 #pragma unroll
       for (int kk = 0; kk < RT / 2; ++kk) {
         if (2 * kk > it) continue;
@@ -340,7 +448,7 @@ __global__ __launch_bounds__(256, 1) void delta_prefill_kernel(DeltaArgs p) {
       }
       const int i = 16 * it + l15;
       if (i < n)
-        *(quad_t*)(p.o + (int64_t)(row0 + ck * DC + i) * p.ldo + (int64_t)h * p.dv + dv0 + 16 * wave + 4 * l4) = to_quad(out[it]);
+        *(quad_t*)(p.o + (int64_t)(row0 + ck * DC) * p.ldo + h * p.dv + dv0 + (uint32_t)(i * (int)p.ldo + 16 * wave + 4 * l4)) = to_quad(out[it]);
     }
     // S <- e^(G_n) S + K~^T diag(e^(G_n - G) rk) U
     const float f = vec[3 * DC];
@@ -352,16 +460,26 @@ __global__ __launch_bounds__(256, 1) void delta_prefill_kernel(DeltaArgs p) {
     for (int kk = 0; kk < RT / 2; ++kk)
 #pragma unroll
       for (int t = 0; t < NS; ++t) {
-        const quad_t a0 = KT::column_quad(kt, 32 * kk, t, l15, l4), a1 = KT::column_quad(kt, 32 * kk + 16, t, l15, l4);
+        const quad_t a0 = KT::column_quad(kt, at, 32 * kk, t, l15, l4), a1 = KT::column_quad(kt, at, 32 * kk + 16, t, l15, l4);
 #pragma unroll
         for (int o = 0; o < NOPND; ++o) S[t] = mma_quads(a0, a1, us[2 * kk][o], us[2 * kk + 1][o], S[t]);
       }
     __syncthreads();
   }
+  if (matrix) {
+    float* m = seg_at(idx) + DK * p.dv + dv0 + 16 * wave + l15;
 #pragma unroll
-  for (int t = 0; t < NS; ++t)
+    for (int t = 0; t < NS; ++t)
 #pragma unroll
-    for (int r = 0; r < 4; ++r) own[(int64_t)(16 * t + r) * p.dv] = S[t][r];
+      for (int r = 0; r < 4; ++r) m[(16 * t + 4 * l4 + r) * DK] = S[t][r];
+  } else if (!OUTPUT) {
+    keep(idx);
+  } else if (idx == nseg - 1) {
+#pragma unroll
+    for (int t = 0; t < NS; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) own[sbase + (uint32_t)((16 * t + r) * p.dv)] = S[t][r];
+  }
 }
 
 // ---- one token per sequence ----
@@ -445,13 +563,25 @@ __global__ __launch_bounds__(4 * DV) void delta_decode_kernel(DeltaDecodeArgs p)
 }
 
 template <int DK>
-static int launch(const DeltaArgs& a, int portions, int n_chunks, hipStream_t s) {
+static int launch(const DeltaArgs& a, int segments, int multi, int n_chunks, hipStream_t s) {
   const int channels = 2 * a.G * DK + a.H * a.dv;
-  hipLaunchKernelGGL(delta_conv_kernel, dim3(n_chunks * (DC / CONV_TOKENS), (channels + 256 * FR - 1) / (256 * FR)), dim3(256), 0, s, a);
+  const dim3 cgrid(n_chunks * (DC / CONV_TOKENS), (channels + 256 * FR - 1) / (256 * FR));
+  switch (a.taps) {
+    case 1: hipLaunchKernelGGL(delta_conv_kernel<1>, cgrid, dim3(256), 0, s, a); break;
+    case 2: hipLaunchKernelGGL(delta_conv_kernel<2>, cgrid, dim3(256), 0, s, a); break;
+    case 3: hipLaunchKernelGGL(delta_conv_kernel<3>, cgrid, dim3(256), 0, s, a); break;
+    case 4: hipLaunchKernelGGL(delta_conv_kernel<4>, cgrid, dim3(256), 0, s, a); break;
+    default: hipLaunchKernelGGL(delta_conv_kernel<0>, cgrid, dim3(256), 0, s, a);
+  }
   hipLaunchKernelGGL((delta_chunk_kernel<DK>), dim3(n_chunks, a.H), dim3(64), 0, s, a);
-  auto k = delta_prefill_kernel<DK>;
+  if (multi) {
+    auto k = delta_prefill_kernel<DK, false>;
+    if (allow_lds(k, DeltaGeom<DK>::LDS)) return LM_EINVAL;
+    hipLaunchKernelGGL(k, dim3(segments, a.H, (a.dv + DK) / 64), dim3(256), DeltaGeom<DK>::LDS, s, a);
+  }
+  auto k = delta_prefill_kernel<DK, true>;
   if (allow_lds(k, DeltaGeom<DK>::LDS)) return LM_EINVAL;
-  hipLaunchKernelGGL(k, dim3(portions, a.H, a.dv / 64), dim3(256), DeltaGeom<DK>::LDS, s, a);
+  hipLaunchKernelGGL(k, dim3(segments, a.H, a.dv / 64), dim3(256), DeltaGeom<DK>::LDS, s, a);
   return launch_status();
 }
 
@@ -462,19 +592,20 @@ using namespace lm;
 extern "C" int lm_delta_chunk_rows(void) { return DC; }
 extern "C" int64_t lm_delta_mat_elems(void) { return MATS; }
 
-extern "C" int lm_delta_prefill(const void* x, int64_t ld, void* o, int64_t ldo, float* state, float* ring, const int* portion,
-                                int portions, const int* chunks, int n_chunks, const float* conv_w, int taps, float qk_eps, float scale,
+extern "C" int lm_delta_prefill(const void* x, int64_t ld, void* o, int64_t ldo, float* state, float* ring, float* seg_state,
+                                const int* portion, const int* chunks, int n_chunks, const int* seg, int segments, int multi,
+                                const float* conv_w, int taps, float qk_eps, float scale,
                                 int64_t ab_col, const float* a_log, const float* dt_bias, void* y, float* norms, void* mats, float* vecs,
                                 int H, int G, int dk, int dv, void* stream) {
-  if (portions <= 0 || n_chunks < portions || H <= 0 || G <= 0 || H % G || dv <= 0 || dv % 64 || taps <= 0 || ld % FR || ldo % 4 || !y ||
+  if (segments <= 0 || n_chunks < segments || (multi && !seg_state) || H <= 0 || G <= 0 || H % G || dv <= 0 || dv % 64 || taps <= 0 || ldo > (1 << 24) || ld % FR || ldo % 4 || !y ||
       !norms || !mats || !vecs)
     return LM_EINVAL;
-  DeltaArgs a{(const elem_t*)x, ld, (elem_t*)o, ldo, state, ring, portion, chunks, conv_w, taps, qk_eps, scale, ab_col, a_log, dt_bias,
+  DeltaArgs a{(const elem_t*)x, ld, (elem_t*)o, ldo, state, ring, portion, chunks, seg, seg_state, conv_w, taps, qk_eps, scale, ab_col, a_log, dt_bias,
               (elem_t*)y, norms, (elem_t*)mats, vecs, H, G, dk, dv};
   hipStream_t s = (hipStream_t)stream;
-  if (dk == 64) return launch<64>(a, portions, n_chunks, s);
-  if (dk == 128) return launch<128>(a, portions, n_chunks, s);
-  if (dk == 256) return launch<256>(a, portions, n_chunks, s);
+  if (dk == 64) return launch<64>(a, segments, multi, n_chunks, s);
+  if (dk == 128) return launch<128>(a, segments, multi, n_chunks, s);
+  if (dk == 256) return launch<256>(a, segments, multi, n_chunks, s);
   return LM_EINVAL;
 }
 

@@ -22,7 +22,7 @@ struct GlaArgs {
   const elem_t* x; int64_t ld;           // row: q [H][dk], k [H][dk], v [H][dv], ...; from low_col on the decays' low-rank input
   elem_t* o; int64_t ldo;                // [tokens][H][dv]
   float* state;                          // [slots][H][dk][dv]
-  float* seg_state;                      // [segments][H][dk][dv]
+  float* seg_state;                      // [segments][H][dk * dv]
   float* seg_decay;                      // [segments][H][dk], powers of two
   const int* seg;                        // [segments][8]: first token, tokens, slot, 1 = starts from zero, index in its entry,
                                          //                segments of the entry, 0, 0
@@ -49,8 +49,10 @@ struct GlaGeom {
   static_assert(NV >= 1 && C * VB % (16 * TH) == 0, "value tile");
 };
 
+constexpr int gla_waves_per_simd(int dk, int waves) { return !SPLIT ? 1 : dk <= 128 ? (waves == 8 ? 4 : 2) : 1; }      // what the registers allow
+
 template <int DK, int NWV, bool OUTPUT>
-__global__ __launch_bounds__(64 * NWV, SPLIT ? 2 : 1) void gla_prefill_kernel(GlaArgs p) {
+__global__ __launch_bounds__(64 * NWV, gla_waves_per_simd(DK, NWV)) void gla_prefill_kernel(GlaArgs p) {
   typedef GlaGeom<DK, NWV> Gm;
   typedef Tile<Gm::KB> KT;
   typedef Tile<Gm::VB> VT;
@@ -65,38 +67,60 @@ __global__ __launch_bounds__(64 * NWV, SPLIT ? 2 : 1) void gla_prefill_kernel(Gl
   const int row0 = sp[0], count = sp[1], slot = sp[2], fresh = sp[3], idx = sp[4], nseg = sp[5];
   if (!OUTPUT && idx == nseg - 1) return;             // nothing follows the last segment
   const int64_t st_stride = (int64_t)DK * p.dv;
-  const int64_t sbase = (int64_t)4 * l4 * p.dv + dv0 + 16 * wave + l15;     // this lane's column, row 4 l4
+  const uint32_t sbase = 4 * l4 * p.dv + dv0 + 16 * wave + l15;     // this lane's column, row 4 l4
   auto store_state = [&](float* s, const f32x4 (&S)[NS]) {
 #pragma unroll
     for (int t = 0; t < NS; ++t)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) s[sbase + (int64_t)(16 * t + r) * p.dv] = S[t][r];
+      for (int r = 0; r < 4; ++r) s[sbase + (uint32_t)((16 * t + r) * p.dv)] = S[t][r];
   };
   auto load_state = [&](const float* s, f32x4 (&S)[NS]) {
 #pragma unroll
     for (int t = 0; t < NS; ++t)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) S[t][r] = s[sbase + (int64_t)(16 * t + r) * p.dv];
+      for (int r = 0; r < 4; ++r) S[t][r] = s[sbase + (uint32_t)((16 * t + r) * p.dv)];
   };
   f32x4 S[NS];
 #pragma unroll
   for (int t = 0; t < NS; ++t) S[t] = zero4();
   float* own = p.state + ((int64_t)slot * p.H + h) * st_stride;
-  auto seg_at = [&](int i) { return p.seg_state + ((int64_t)(sg - idx + i) * p.H + h) * st_stride; };
+  // states between the passes lie as the accumulators hold them: [segment][head][16 columns][NS][lane][4]
+  auto seg_at = [&](int i) {
+    return (f32x4*)(p.seg_state + ((int64_t)(sg - idx + i) * p.H + h) * st_stride + (int64_t)(dv0 + 16 * wave) * DK) + lane;
+  };
+  auto keep = [&](int i) {
+    f32x4* s = seg_at(i);
+#pragma unroll
+    for (int t = 0; t < NS; ++t) s[64 * t] = S[t];
+  };
+  auto recall = [&](int i) {
+    const f32x4* s = seg_at(i);
+#pragma unroll
+    for (int t = 0; t < NS; ++t) S[t] = s[64 * t];
+  };
   if (idx == 0) {
-    if (OUTPUT && nseg > 1) load_state(seg_at(nseg - 1), S);      // kept by the first pass: the last segment replaces the slot's state
+    if (OUTPUT && nseg > 1) recall(nseg - 1);         // kept by the first pass: the last segment replaces the slot's state
     else if (!fresh) load_state(own, S);
-    if (!OUTPUT) store_state(seg_at(nseg - 1), S);
+    if (!OUTPUT) keep(nseg - 1);
   } else if (OUTPUT) {
     // ((s_0 d_1 + s_1) d_2 + s_2) ..., d the segments' decays
-    load_state(seg_at(0), S);
+    recall(0);
     for (int i = 1; i < idx; ++i) {
-      const float *d = p.seg_decay + ((int64_t)(sg - idx + i) * p.H + h) * DK + 4 * l4, *s = seg_at(i);
+      const float* d = p.seg_decay + ((int64_t)(sg - idx + i) * p.H + h) * DK + 4 * l4;
+      const f32x4* s = seg_at(i);
+      constexpr int B = NS < 4 ? NS : 4;
 #pragma unroll
-      for (int t = 0; t < NS; ++t) {
-        const f32x4 f = *(const f32x4*)(d + 16 * t);
+      for (int t0 = 0; t0 < NS; t0 += B) {
+        f32x4 f[B], a[B];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) S[t][r] = S[t][r] * __builtin_amdgcn_exp2f(f[r]) + s[sbase + (int64_t)(16 * t + r) * p.dv];
+        for (int t = 0; t < B; ++t) {
+          f[t] = *(const f32x4*)(d + 16 * (t0 + t));
+          a[t] = s[64 * (t0 + t)];
+        }
+#pragma unroll
+        for (int t = 0; t < B; ++t)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) S[t0 + t][r] = S[t0 + t][r] * __builtin_amdgcn_exp2f(f[t][r]) + a[t][r];
       }
     }
   }
@@ -104,42 +128,65 @@ __global__ __launch_bounds__(64 * NWV, SPLIT ? 2 : 1) void gla_prefill_kernel(Gl
   const elem_t* src = p.x + (int64_t)row0 * p.ld;
   const int64_t qo = (int64_t)h * DK, ko = (int64_t)(p.H + h) * DK, vo = (int64_t)2 * p.H * DK + (int64_t)h * p.dv + dv0;
   frag_t rq[OUTPUT ? Gm::NQ : 1], rk[Gm::NQ], rv[Gm::NV];
-  auto fetch = [&](int c0) {
+  const int ldx = (int)p.ld;
+  auto fetch = [&](int c0) {                           // (rows past the end: the last one's values meet k' = q' = 0)
+    const elem_t* base = src + (int64_t)c0 * p.ld;     // the same for all lanes; the lanes' offsets fit 32 bits
+    const int last = count - 1 - c0;
 #pragma unroll
     for (int i = 0; i < Gm::NQ; ++i) {
       const int sl = Gm::TH * i + tid, r = sl / KT::NS, s = sl % KT::NS;
-      const bool in = c0 + r < count && (Gm::QWHOLE || r < C);
-      const elem_t* a = src + (int64_t)(in ? c0 + r : 0) * p.ld + s * FR;
-      if constexpr (OUTPUT) rq[i] = in ? *(const frag_t*)(a + qo) : frag_t{};
-      rk[i] = in ? *(const frag_t*)(a + ko) : frag_t{};
+      const uint32_t off = min(r, last) * ldx + s * FR;
+      if constexpr (OUTPUT) rq[i] = *(const frag_t*)(base + qo + off);
+      rk[i] = *(const frag_t*)(base + ko + off);
     }
 #pragma unroll
     for (int i = 0; i < Gm::NV; ++i) {
       const int sl = Gm::TH * i + tid, r = sl / VT::NS, s = sl % VT::NS;
-      const bool in = c0 + r < count;
-      rv[i] = in ? *(const frag_t*)(src + (int64_t)(c0 + r) * p.ld + vo + s * FR) : frag_t{};
+      rv[i] = *(const frag_t*)(base + vo + (uint32_t)(min(r, last) * ldx + s * FR));
     }
   };
+  // the decays' input: its first 64 columns (all of them, as a rule) are requested one chunk ahead
+  constexpr int NL = 64 / KSTEP;
+  frag_t rl[RT][NL];
+  auto fetch_low = [&](int c0) {
+    const elem_t* base = src + (int64_t)c0 * p.ld + p.low_col;
+    const int last = count - 1 - c0;
+#pragma unroll
+    for (int u = 0; u < RT; ++u)
+#pragma unroll
+      for (int s = 0; s < NL; ++s) rl[u][s] = *(const frag_t*)(base + (uint32_t)(min(16 * u + l15, last) * ldx + s * KSTEP + FR * l4));
+  };
   float total = 0.f;                                  // !OUTPUT: of channel tid, the segment's decay so far
+  fetch_low(0);
   fetch(0);
+  typename KT::Offsets at(l15, l4);
   for (int c0 = 0, n; c0 < count; c0 += n) {
+    at.forget();
     // ---- B: tokens are the rows, channels the columns of the product tiles ----
     int end = C;                                      // first place whose B is below the limit
+#pragma unroll 1
     for (int cb = wave; cb < NS; cb += NWV) {
-      const int ch = h * DK + 16 * cb + l15;
-      const elem_t* ap = p.a2 + (int64_t)ch * p.rp + FR * l4;
-      const float bias = p.bias[ch];
+      uint32_t ch = 16 * cb + l15;
+      asm volatile("" : "+v"(ch));                    // (no addresses kept from chunk to chunk)
+      const elem_t* ap = p.a2 + (int64_t)h * DK * p.rp;
+      const uint32_t ao = ch * p.rp + FR * l4;
+      frag_t a[64 / KSTEP];
+#pragma unroll
+      for (int s = 0; s < 64 / KSTEP; ++s) a[s] = *(const frag_t*)(ap + (ao + s * KSTEP));
+      const float bias = (p.bias + h * DK)[ch];
       float carry = 0.f;
 #pragma unroll
       for (int u = 0; u < RT; ++u) {
-        const elem_t* lp = src + (int64_t)min(c0 + 16 * u + l15, count - 1) * p.ld + p.low_col + FR * l4;
         f32x4 z = zero4();
-        for (int s = 0; s < p.rp; s += KSTEP) z = mma(*(const frag_t*)(lp + s), *(const frag_t*)(ap + s), z);
+#pragma unroll
+        for (int s = 0; s < 64 / KSTEP; ++s) z = mma(rl[u][s], a[s], z);
+        for (int s = 64; s < p.rp; s += KSTEP)
+          z = mma(*(const frag_t*)(src + (int64_t)c0 * p.ld + p.low_col + (uint32_t)(min(16 * u + l15, count - 1 - c0) * ldx + s + FR * l4)),
+                  *(const frag_t*)(ap + (ao + s)), z);
         float sum = 0.f;
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const bool in = c0 + 16 * u + 4 * l4 + r < count;
-          sum += in ? log_decay(z[r] + bias, p.inv_tau) : 0.f;
+          sum += log_decay(z[r] + bias, p.inv_tau);   // (places past the end follow all others and are not used)
           z[r] = sum;                                 // running sum within the lane
         }
         float before = 0.f, all = 0.f;                // of the lanes in front, of the block
@@ -152,15 +199,16 @@ __global__ __launch_bounds__(64 * NWV, SPLIT ? 2 : 1) void gla_prefill_kernel(Gl
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int i = 16 * u + 4 * l4 + r;
-          const float v = z[r] + (before + carry);
-          if (v < -LIMIT) end = min(end, i);
-          *(float*)(bb + i * Gm::BB + (16 * cb + l15) * 4) = v;
+          *(float*)(bb + i * Gm::BB + (16 * cb + l15) * 4) = z[r] + (before + carry);
         }
         carry += all;
       }
+      if (__builtin_amdgcn_ballot_w64(carry < -LIMIT) != 0) {      // some channel's B passes the limit (B only falls)
+#pragma unroll 1
+        for (int i = C - 1; i >= 0; --i)
+          if (__builtin_amdgcn_ballot_w64(*(const float*)(bb + i * Gm::BB + (16 * cb + l15) * 4) < -LIMIT) != 0) end = min(end, i);
+      }
     }
-#pragma unroll
-    for (int m = 32; m > 0; m >>= 1) end = min(end, __shfl_xor(end, m, 64));
     if (lane == 0) ends[wave] = end;
     __syncthreads();
     n = min(C, count - c0);
@@ -205,7 +253,6 @@ __global__ __launch_bounds__(64 * NWV, SPLIT ? 2 : 1) void gla_prefill_kernel(Gl
       tot[tid] = __builtin_amdgcn_exp2f(b);
       total += b;
     }
-    if (c0 + n < count) fetch(c0 + n);
     __syncthreads();
 
     quad_t vq[RT];                                     // V, column l15 of this wave, all tokens of the chunk
@@ -222,12 +269,13 @@ __global__ __launch_bounds__(64 * NWV, SPLIT ? 2 : 1) void gla_prefill_kernel(Gl
         if (u <= it) {
 #pragma unroll
           for (int k = 0; k < DK / KSTEP; ++k) {
-            const frag_t k0 = KT::frag(kt, 16 * u + l15, 4 * k + l4), q0 = KT::frag(qt, i, 4 * k + l4);
+            const frag_t k0 = KT::frag(kt, at, 16 * u, k), q0 = KT::frag(qt, at, 16 * it, k);
             s = mma(k0, q0, s);
             if constexpr (SPLIT) {
-              s = mma(k0, KT::frag(qt + C * Gm::KB, i, 4 * k + l4), s);
-              s = mma(KT::frag(kt + C * Gm::KB, 16 * u + l15, 4 * k + l4), q0, s);
+              s = mma(k0, KT::frag(qt + C * Gm::KB, at, 16 * it, k), s);
+              s = mma(KT::frag(kt + C * Gm::KB, at, 16 * u, k), q0, s);
             }
+            if (k % 2 == 1) __builtin_amdgcn_sched_barrier(0);      // (registers: not all operands at once)
           }
           if (u == it) {
 #pragma unroll
@@ -239,6 +287,7 @@ __global__ __launch_bounds__(64 * NWV, SPLIT ? 2 : 1) void gla_prefill_kernel(Gl
 #pragma unroll
         for (int o = 0; o < NOPND; ++o) *(quad_t*)(pt + (o * C + i) * Gm::PB + (16 * u + 4 * l4) * Gm::ES) = q[o];
       }
+      __builtin_amdgcn_sched_barrier(0);
       // what the state in front of the chunk contributes: O^T = S^T Q'^T, rows of this wave's 16 columns
       f32x4 out[RT];
 #pragma unroll
@@ -250,14 +299,15 @@ __global__ __launch_bounds__(64 * NWV, SPLIT ? 2 : 1) void gla_prefill_kernel(Gl
         split_quad(S[t + 1], a1);
 #pragma unroll
         for (int it = 0; it < RT; ++it) {
-          const quad_t b0 = KT::quad(qt, 16 * it + l15, t, l4), b1 = KT::quad(qt, 16 * it + l15, t + 1, l4);
+          const quad_t b0 = KT::quad(qt, at, 16 * it, t), b1 = KT::quad(qt, at, 16 * it, t + 1);
 #pragma unroll
           for (int o = 0; o < NOPND; ++o) out[it] = mma_quads(a0[o], a1[o], b0, b1, out[it]);
           if constexpr (SPLIT) {
             const uint8_t* ql = qt + C * Gm::KB;
-            out[it] = mma_quads(a0[0], a1[0], KT::quad(ql, 16 * it + l15, t, l4), KT::quad(ql, 16 * it + l15, t + 1, l4), out[it]);
+            out[it] = mma_quads(a0[0], a1[0], KT::quad(ql, at, 16 * it, t), KT::quad(ql, at, 16 * it, t + 1), out[it]);
           }
         }
+        __builtin_amdgcn_sched_barrier(0);      // (registers: not all operands at once)
       }
       __syncthreads();
 #pragma unroll
@@ -274,9 +324,10 @@ __global__ __launch_bounds__(64 * NWV, SPLIT ? 2 : 1) void gla_prefill_kernel(Gl
         }
         const int i = 16 * it + l15;
         if (i < n)
-          *(quad_t*)(p.o + (int64_t)(row0 + c0 + i) * p.ldo + (int64_t)h * p.dv + dv0 + 16 * wave + 4 * l4) = to_quad(out[it]);
+          *(quad_t*)(p.o + (int64_t)(row0 + c0) * p.ldo + h * p.dv + dv0 + (uint32_t)(i * (int)p.ldo + 16 * wave + 4 * l4)) = to_quad(out[it]);
       }
     }
+    if (c0 + n < count) fetch_low(c0 + n);
     // S <- e^(B_n) (S + K'^T V)
 #pragma unroll
     for (int t = 0; t < NS; ++t) {
@@ -285,15 +336,18 @@ __global__ __launch_bounds__(64 * NWV, SPLIT ? 2 : 1) void gla_prefill_kernel(Gl
 #pragma unroll
         for (int o = 0; o < NOPND; ++o) {
           const uint8_t* k = kt + o * C * Gm::KB;
-          S[t] = mma_quads(KT::column_quad(k, 32 * kk, t, l15, l4), KT::column_quad(k, 32 * kk + 16, t, l15, l4), vq[2 * kk],
+          S[t] = mma_quads(KT::column_quad(k, at, 32 * kk, t, l15, l4), KT::column_quad(k, at, 32 * kk + 16, t, l15, l4), vq[2 * kk],
                            vq[2 * kk + 1], S[t]);
         }
       S[t] *= *(const f32x4*)(tot + 16 * t + 4 * l4);
+      if (t % 2 == 1) __builtin_amdgcn_sched_barrier(0);
     }
+    __builtin_amdgcn_sched_barrier(0);
+    if (c0 + n < count) fetch(c0 + n);                 // (here and not earlier: registers)
     // (no barrier: the next chunk writes B first, which nobody reads any more, and then waits)
   }
   if (!OUTPUT) {
-    store_state(seg_at(idx), S);
+    keep(idx);
     if (tid < DK && dv0 == 0) p.seg_decay[((int64_t)sg * p.H + h) * DK + tid] = total;
   } else if (idx == nseg - 1) {
     store_state(own, S);
@@ -389,8 +443,8 @@ using namespace lm;
 extern "C" int lm_gla_prefill(const void* x, int64_t ld, void* o, int64_t ldo, float* state, float* seg_state, float* seg_decay,
                               const int* seg, int segments, int multi, int64_t low_col, const void* a2, const float* bias, int rp,
                               float inv_tau, float scale, int H, int dk, int dv, void* stream) {
-  if (segments <= 0 || H <= 0 || dv <= 0 || dv % 64 || (multi && (!seg_state || !seg_decay)) || ld % FR || ldo % 4 || low_col % FR ||
-      rp <= 0 || rp % KSTEP || !(inv_tau > 0.f))
+  if (segments <= 0 || H <= 0 || dv <= 0 || dv % 64 || (multi && (!seg_state || !seg_decay)) || ld > (1 << 24) || ldo > (1 << 24) || ld % FR || ldo % 4 || low_col % FR ||
+      rp < 64 || rp % 64 || !(inv_tau > 0.f))
     return LM_EINVAL;
   GlaArgs a{(const elem_t*)x, ld, (elem_t*)o, ldo, state, seg_state, seg_decay, seg, low_col, (const elem_t*)a2, bias, rp, inv_tau, scale,
             H, dv};

@@ -193,20 +193,40 @@ __global__ __launch_bounds__(ROW_THREADS) void gated_head_rms_kernel(elem_t* out
   }
 }
 
-// gated unit of rows in alternating blocks of 16 gate and 16 up channels
-__global__ __launch_bounds__(ROW_THREADS) void glu_kernel(elem_t* out, int64_t ldo, const elem_t* x, int64_t ldx, const float* bias, int n,
-                                                          int act) {
-  const int64_t t = blockIdx.x;
-  for (int c = FR * (int)threadIdx.x; c < n; c += FR * ROW_THREADS) {
-    const int s = 32 * (c >> 4) + (c & 15);
-    const frag_t g = *(const frag_t*)(x + t * ldx + s), u = *(const frag_t*)(x + t * ldx + s + 16);
-    frag_t r;
+// gated unit of rows in alternating blocks of 16 gate and 16 up channels; a thread's channels of GLU_ROWS rows
+constexpr int GLU_ROWS = 16;
+
+__global__ __launch_bounds__(ROW_THREADS) void glu_kernel(elem_t* out, int64_t ldo, const elem_t* x, int64_t ldx, const float* bias, int rows,
+                                                          int n, int act) {
+  const int c = FR * (int)(blockIdx.x * ROW_THREADS + threadIdx.x), s = 32 * (c >> 4) + (c & 15);
+  if (c >= n) return;
+  float bg[FR], bu[FR];
 #pragma unroll
-    for (int e = 0; e < FR; ++e) {
-      const float a = (float)g[e] + (bias ? bias[s + e] : 0.f), b = (float)u[e] + (bias ? bias[s + 16 + e] : 0.f);
-      r[e] = (elem_t)((act == LM_ACT_GELU_TANH ? gelu_tanh(a) : silu(a)) * b);
+  for (int e = 0; e < FR; ++e) {
+    bg[e] = bias ? bias[s + e] : 0.f;
+    bu[e] = bias ? bias[s + 16 + e] : 0.f;
+  }
+  const int64_t t0 = (int64_t)GLU_ROWS * blockIdx.y, t1 = t0 + GLU_ROWS < rows ? t0 + GLU_ROWS : rows;
+  constexpr int B = 4;      // rows in flight
+  for (int64_t t = t0; t < t1; t += B) {
+    frag_t g[B], u[B];
+#pragma unroll
+    for (int b = 0; b < B; ++b) {
+      const elem_t* xr = x + (t + b < t1 ? t + b : t1 - 1) * ldx + s;
+      g[b] = *(const frag_t*)xr;
+      u[b] = *(const frag_t*)(xr + 16);
     }
-    *(frag_t*)(out + t * ldo + c) = r;
+#pragma unroll
+    for (int b = 0; b < B; ++b) {
+      if (t + b >= t1) break;
+      frag_t r;
+#pragma unroll
+      for (int e = 0; e < FR; ++e) {
+        const float a = (float)g[b][e] + bg[e];
+        r[e] = (elem_t)((act == LM_ACT_GELU_TANH ? gelu_tanh(a) : silu(a)) * ((float)u[b][e] + bu[e]));
+      }
+      *(frag_t*)(out + (t + b) * ldo + c) = r;
+    }
   }
 }
 
@@ -348,7 +368,8 @@ extern "C" int lm_gated_head_rms(void* out, int64_t ldo, const void* o, int64_t 
 
 extern "C" int lm_glu(void* out, int64_t ldo, const void* x, int64_t ldx, const float* bias, int rows, int n, int act, void* stream) {
   if (rows <= 0 || n <= 0 || n % 16 || ldo % FR || ldx % FR || (act != LM_ACT_SILU && act != LM_ACT_GELU_TANH)) return LM_EINVAL;
-  hipLaunchKernelGGL(glu_kernel, dim3(rows), dim3(ROW_THREADS), 0, (hipStream_t)stream, (elem_t*)out, ldo, (const elem_t*)x, ldx, bias, n,
+  const dim3 grid((n + ROW_THREADS * FR - 1) / (ROW_THREADS * FR), (rows + GLU_ROWS - 1) / GLU_ROWS);
+  hipLaunchKernelGGL(glu_kernel, grid, dim3(ROW_THREADS), 0, (hipStream_t)stream, (elem_t*)out, ldo, (const elem_t*)x, ldx, bias, rows, n,
                      act);
   return launch_status();
 }

@@ -99,7 +99,9 @@ class BatchBuilder:
                     chunks += [len(ports) - 1] * nc
                 ns = -(-n // seg_len)
                 multi |= ns > 1
-                segs += [(at + s * seg_len, min(seg_len, n - s * seg_len), e.seq.slot, int(p0 == 0), s, ns, 0, 0) for s in range(ns)]
+                ck = (ports[-1][4], seg_len // self.chunk) if self.chunk else (0, 0)
+                segs += [(at + s * seg_len, min(seg_len, n - s * seg_len), e.seq.slot, int(p0 == 0), s, ns, ck[0] + s * ck[1], 0)
+                         for s in range(ns)]
             for w in e.want:
                 rows.append(at + w)
                 wanted.append((i, w))

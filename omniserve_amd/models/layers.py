@@ -461,7 +461,7 @@ class GatedLinearAttention(Mixer):
         self.bias = bias.view(-1)
         self.w_out = pad_in_heads(w.matrix("o", width, H * s.vdim), H, s.vdim, W)
         self.norm = w.vector("norm", s.vdim, self.dv)
-        self.segment_workgroups = H * self.dv // 64
+        self.segment_workgroups = max(1, H * self.dv // 128)
 
     def state_shapes(self):
         return [(self.s.heads, self.dk, self.dv)]
@@ -505,6 +505,7 @@ class DeltaRule(Mixer):
         self.a_log, self.dt_bias = w.vector("A_log", H), w.vector("dt_bias", H)
         self.w_out = pad_in_heads(w.matrix("o", width, H * s.vdim), H, s.vdim, W)
         self.norm = w.vector("norm", s.vdim, self.dv)
+        self.segment_workgroups = H * self.dv // 64
 
     def state_shapes(self):
         return [(self.s.heads, self.dk, self.dv), (self.s.taps, self.g0)]
@@ -516,7 +517,7 @@ class DeltaRule(Mixer):
         rule = (self.conv, s.unit_eps, s.dim ** -0.5, self.ab0, self.a_log, self.dt_bias)
         size = (s.heads, s.kv_heads, self.dk, self.dv)
         if n:
-            ops.delta_prefill(x[:n], o[:n], state, ring, b.portions, b.chunks, *rule, *size)
+            ops.delta_prefill(x[:n], o[:n], state, ring, b.portions, b.chunks, b.segments, b.multi_segment, *rule, *size)
             ops.gated_head_rms(o[:n], o[:n], x[:n, self.g0:], self.norm, s.heads, self.dv, s.vdim, self.eps, "silu")
         if b.n_decode:
             ops.delta_decode(x[n:], o[n:], state, ring, b.state_slot, b.pos[n:], *rule, self.g0, self.norm, s.vdim, self.eps, *size)

@@ -68,6 +68,12 @@ def test_batch_tables_of_chunks_and_expansions():
     assert [p[:4] for p in ports] == [[0, 33, seqs[0].slot, 1], [33, 64, seqs[1].slot, 0], [97, 2, seqs[2].slot, 0], [99, 40, seqs[4].slot, 0]]
     assert [p[4:7] for p in ports] == [[0, 2, 0], [2, 2, 100], [4, 1, 63], [5, 2, 300]]
     assert chunks == [0, 0, 1, 1, 2, 3, 3]
+    long = cache.open()
+    cache.reserve(long, 700)
+    s, _ = builder.build([Entry(seqs[3], [0, 0], []), Entry(long, [0] * 700, [])])
+    assert s.multi_segment and s.segment_len == 256
+    assert [x[:7] for x in s.segments.tolist()] == [[0, 2, seqs[3].slot, 0, 0, 1, 0]] + [
+        [2 + 256 * i, n, long.slot, 1, i, 3, 1 + 8 * i] for i, n in enumerate((256, 256, 188))]
     # pages: 1, 3, 2, 6; at most 4 at once, one portion at least
     assert b.expansions == ((0, 4, 0, 2), (4, 2, 2, 1), (6, 6, 3, 1))
     pages, table = b.context_pages.tolist(), b.context_table.tolist()

@@ -144,9 +144,10 @@ def test_delta_mixer(name, dtype):
     m = OneMixer(DELTA[name], 96, dtype, seed=5)
     h = inputs(333, 96, 6)
     want = m.oracle(h)
-    for sizes in ([333], [31, 2, 64, 1, 1, 130], [65, 63], [2], [3, 1, 1], [1]):
-        e = errors(m.run(h, sizes), want)
-        assert e.max() < TOL[dtype], (sizes, e.argmax(), e.max())
+    for sizes, seg in (([333], None), ([333], 64), ([333], 128), ([31, 2, 64, 1, 1, 130], 64), ([65, 63], None), ([2], None), ([3, 1, 1], None),
+                       ([1], None)):
+        e = errors(m.run(h, sizes, seg_len=seg), want)
+        assert e.max() < TOL[dtype], (sizes, seg, e.argmax(), e.max())
 
 
 @pytest.mark.parametrize("dtype", DTYPES, ids=str)
@@ -182,9 +183,9 @@ def test_delta_rule_with_one_key_for_all_tokens(dtype):
     h = inputs(400, W, 10)
     h[:, 0] = 3.0
     want = m.oracle(h)
-    for sizes in ([400], [130, 2, 64], [1]):
-        e = errors(m.run(h, sizes), want)
-        assert e.max() < 2 * TOL[dtype], (sizes, e.argmax(), e.max())
+    for sizes, seg in (([400], None), ([400], 64), ([130, 2, 64], None), ([1], None)):
+        e = errors(m.run(h, sizes, seg_len=seg), want)
+        assert e.max() < 2 * TOL[dtype], (sizes, seg, e.argmax(), e.max())
 
 
 @pytest.mark.parametrize("dtype", DTYPES, ids=str)
