@@ -13,8 +13,8 @@
 //   prefill   one workgroup per (segment, head, 64 value columns) walks the chunks: R = V - diag(e^G rk) K~ S, U = T R, the outputs
 //             and the next state.  S stays in MFMA accumulators; every result tile is the next product's operand as it lies.
 // Long portions are cut into segments that run in parallel.  A segment takes a state S to M S + C: a first pass forms C (the segment
-// from a zero state) and, as dk more columns, M (the segment without values, from the identity); the second pass starts every segment
-// from the states these give.
+// from a zero state) and, as dk more columns, M (the segment without values, from the identity); `chain` turns the C into the states
+// behind the segments, from which the second pass starts.
 // f32 factors (S, R, U, T, P) enter the bf16 products as two bf16 operands each; of two such factors the product of the two low
 // parts is dropped.
 #include "lm_state.h"
@@ -136,7 +136,7 @@ __global__ __launch_bounds__(64) void delta_chunk_kernel(DeltaArgs p) {
   __shared__ __attribute__((aligned(16))) float A[DC][AP];
   __shared__ float Gs[DC], be[DC], rqs[DC], rks[DC];
   const int lane = threadIdx.x, l15 = lane & 15, l4 = lane >> 4;
-  const int ck = blockIdx.x, h = blockIdx.y, g = h / (p.H / p.G);
+  const int ck = blockIdx.y, h = blockIdx.x, g = h / (p.H / p.G);
   const int* pp = p.portion + 8 * p.chunks[ck];
   const int first = pp[0], count = pp[1], slot = pp[2], nch = pp[5], pos0 = pp[6], index = ck - pp[4];
   const int t0 = index * DC, n = min(DC, count - t0);
@@ -172,22 +172,31 @@ __global__ __launch_bounds__(64) void delta_chunk_kernel(DeltaArgs p) {
   __syncthreads();
   elem_t* mt = p.mats + ((int64_t)ck * p.H + h) * MATS;
   elem_t* mp = mt + NOPND * DC * DC;
-  const elem_t* yq = p.y + (int64_t)(first + t0) * channels + (int64_t)g * DK + FR * l4;
+  const elem_t* yq = p.y + (int64_t)(first + t0) * channels + (int64_t)g * DK;
   const elem_t* yk = yq + (int64_t)p.G * DK;
-  for (int u = 0; u < RT; ++u) {                 // keys j of block u against rows i of blocks it >= u (and the zeros beside them)
-    frag_t kf[NKF];
-    const int64_t ju = min(16 * u + l15, n - 1);
+  frag_t kf[RT][NKF], qf[2][NKF];                // all keys, the queries one block ahead
+  auto row_at = [&](int blk) { return (uint32_t)(min(16 * blk + l15, n - 1) * channels + FR * l4); };
 #pragma unroll
-    for (int s = 0; s < NKF; ++s) kf[s] = *(const frag_t*)(yk + ju * channels + s * KSTEP);
-    for (int it = 0; it < RT; ++it) {
+  for (int u = 0; u < RT; ++u)
+#pragma unroll
+    for (int s = 0; s < NKF; ++s) kf[u][s] = *(const frag_t*)(yk + (row_at(u) + s * KSTEP));
+#pragma unroll
+  for (int s = 0; s < NKF; ++s) qf[0][s] = *(const frag_t*)(yq + (row_at(0) + s * KSTEP));
+#pragma unroll
+  for (int it = 0; it < RT; ++it) {              // rows i of block it against keys j of blocks u <= it (and the zeros beside them)
+    if (it + 1 < RT) {
+#pragma unroll
+      for (int s = 0; s < NKF; ++s) qf[(it + 1) & 1][s] = *(const frag_t*)(yq + (row_at(it + 1) + s * KSTEP));
+    }
+#pragma unroll
+    for (int u = 0; u < RT; ++u) {
       const int i = 16 * it + l15, j = 16 * u + 4 * l4;
       f32x4 kk = zero4(), qk = zero4();
-      if (it >= u) {
-        const int64_t ir = min(i, n - 1);
+      if (u <= it) {
 #pragma unroll
         for (int s = 0; s < NKF; ++s) {
-          kk = mma(kf[s], *(const frag_t*)(yk + ir * channels + s * KSTEP), kk);
-          qk = mma(kf[s], *(const frag_t*)(yq + ir * channels + s * KSTEP), qk);
+          kk = mma(kf[u][s], kf[it][s], kk);
+          qk = mma(kf[u][s], qf[it & 1][s], qk);
         }
       }
 #pragma unroll
@@ -244,19 +253,20 @@ __global__ __launch_bounds__(64) void delta_chunk_kernel(DeltaArgs p) {
 }
 
 // ---- the recurrence over a portion's chunks ----
-template <int DK>
+template <int DK, bool OUTPUT>
 struct DeltaGeom {
   static constexpr int NWV = 4, TH = 256, DVB = 64, ES = (int)sizeof(elem_t);
   static constexpr int KB = DK * ES, VB = DVB * ES, PB = DC * ES + 16;
-  static constexpr int Q0 = 0, K0 = DC * KB, V0 = 2 * DC * KB, M0 = V0 + DC * VB, S0 = M0 + 2 * NOPND * DC * PB, LDS = S0 + 4 * DC * 4;
+  static constexpr int Q0 = 0, K0 = OUTPUT ? DC * KB : 0, V0 = K0 + DC * KB, M0 = V0 + DC * VB, S0 = M0 + (OUTPUT ? 2 : 1) * NOPND * DC * PB,
+                       LDS = S0 + 4 * DC * 4;
   static constexpr int NQ = DC * KB / (16 * TH), NV = DC * VB / (16 * TH);
-  static constexpr int MR = DC * ES / 16, NM = 2 * NOPND * DC * MR / TH;      // 16-byte pieces of a matrix row, per thread
-  static_assert(NQ >= 1 && NV >= 1 && NM >= 1 && 2 * NOPND * DC * MR % TH == 0, "loads");
+  static constexpr int MR = DC * ES / 16, NM = (OUTPUT ? 2 : 1) * NOPND * DC * MR / TH;      // 16-byte pieces of a matrix row, per thread
+  static_assert(NQ >= 1 && NV >= 1 && NM >= 1 && NOPND * DC * MR % TH == 0, "loads");
 };
 
 template <int DK, bool OUTPUT>
-__global__ __launch_bounds__(256, SPLIT && DK <= 128 ? 2 : 1) void delta_prefill_kernel(DeltaArgs p) {
-  typedef DeltaGeom<DK> Gm;
+__global__ __launch_bounds__(256, !SPLIT || DK > 128 ? 1 : OUTPUT ? 2 : 3) void delta_prefill_kernel(DeltaArgs p) {
+  typedef DeltaGeom<DK, OUTPUT> Gm;
   typedef Tile<Gm::KB> KT;
   typedef Tile<Gm::VB> VT;
   constexpr int NS = DK / 16, RT = DC / 16, MP = NOPND * DC * Gm::PB;      // MP: bytes of one matrix
@@ -305,38 +315,12 @@ __global__ __launch_bounds__(256, SPLIT && DK <= 128 ? 2 : 1) void delta_prefill
     }
     if (!OUTPUT) keep(nseg - 1);
   } else if (OUTPUT) {
-    recall(0);
-    for (int i = 1; i < idx; ++i) {       // S <- M_i S + C_i
-      const float* m = seg_at(i) + DK * p.dv;
-      const f32x4* c = seg_cols(i);
-      f32x4 N[NS];
-#pragma unroll
-      for (int t = 0; t < NS; ++t) N[t] = c[64 * t];
-#pragma unroll
-      for (int k = 0; k < NS; k += 2) {
-        quad_t s0[NOPND], s1[NOPND];
-        split_quad(S[k], s0);
-        split_quad(S[k + 1], s1);
-#pragma unroll
-        for (int t = 0; t < NS; ++t) {
-          const float* row = m + (uint32_t)((16 * t + l15) * DK + 16 * k + 4 * l4);
-          quad_t a0[NOPND], a1[NOPND];
-          split_quad(*(const f32x4*)row, a0);
-          split_quad(*(const f32x4*)(row + 16), a1);
-#pragma unroll
-          for (int o = 0; o < NOPND; ++o) N[t] = mma_quads(a0[0], a1[0], s0[o], s1[o], N[t]);
-          if constexpr (SPLIT) N[t] = mma_quads(a0[1], a1[1], s0[0], s1[0], N[t]);
-        }
-      }
-#pragma unroll
-      for (int t = 0; t < NS; ++t) S[t] = N[t];
-    }
+    recall(idx - 1);                      // delta_chain_kernel has left the state behind every segment there
   }
 
   const elem_t* src = p.y + (int64_t)row0 * channels;
   const int qo = g * DK, ko = (p.G + g) * DK, vo = 2 * p.G * DK + h * p.dv + dv0;
-  constexpr int NM = OUTPUT ? Gm::NM : Gm::NM / 2;      // (T comes first)
-  frag_t rq[OUTPUT ? Gm::NQ : 1], rk[Gm::NQ], rv[Gm::NV], rm[NM];
+  frag_t rq[OUTPUT ? Gm::NQ : 1], rk[Gm::NQ], rv[Gm::NV], rm[Gm::NM];      // (of the matrices T comes first)
   float rvec = 0.f;
   auto fetch = [&](int ck) {              // addresses: a base all lanes share, 32-bit offsets
     const elem_t* base = src + (int64_t)ck * DC * channels;
@@ -355,7 +339,7 @@ __global__ __launch_bounds__(256, SPLIT && DK <= 128 ? 2 : 1) void delta_prefill
     }
     const int64_t block = (int64_t)(ck0 + ck) * p.H + h;
 #pragma unroll
-    for (int i = 0; i < NM; ++i) rm[i] = *(const frag_t*)(p.mats + block * MATS + (uint32_t)((Gm::TH * i + tid) * FR));
+    for (int i = 0; i < Gm::NM; ++i) rm[i] = *(const frag_t*)(p.mats + block * MATS + (uint32_t)((Gm::TH * i + tid) * FR));
     if (tid < 4 * DC) rvec = (p.vecs + block * 4 * DC)[(uint32_t)tid];
   };
   static_assert(4 * DC <= Gm::TH, "one factor per thread");
@@ -376,7 +360,7 @@ __global__ __launch_bounds__(256, SPLIT && DK <= 128 ? 2 : 1) void delta_prefill
       *(frag_t*)(vt + VT::slot(sl / VT::NS, sl % VT::NS)) = rv[i];
     }
 #pragma unroll
-    for (int i = 0; i < NM; ++i) {
+    for (int i = 0; i < Gm::NM; ++i) {
       const int sl = Gm::TH * i + tid;
       *(frag_t*)(mt + (sl / Gm::MR) * Gm::PB + (sl % Gm::MR) * 16) = rm[i];
     }
@@ -482,6 +466,61 @@ __global__ __launch_bounds__(256, SPLIT && DK <= 128 ? 2 : 1) void delta_prefill
   }
 }
 
+// ---- from a portion's segments (M_i, C_i) to the states behind them, S_i = M_i S_(i-1) + C_i, in place of C_i.  One workgroup per
+// 16 columns; a wave owns a quarter of the rows, the operands of S pass through LDS ----
+template <int DK>
+__global__ __launch_bounds__(256) void delta_chain_kernel(DeltaArgs p) {
+  constexpr int NS = DK / 16, TB = NS / 4;
+  __shared__ __attribute__((aligned(16))) quad_t sq[NOPND][NS][64];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l15 = lane & 15, l4 = lane >> 4;
+  const int sg = blockIdx.z, h = blockIdx.y, nseg = p.seg[8 * sg + 5];      // (those with work are neighbours: on all XCDs)
+  if (p.seg[8 * sg + 4] != 0 || nseg < 3) return;
+  const int64_t stride = (int64_t)DK * (p.dv + DK);
+  float* at = p.seg_state + ((int64_t)sg * p.H + h) * stride;
+  const int64_t next = stride * p.H;                     // to the next segment's
+  const uint32_t c0 = 16 * blockIdx.x * DK + 64 * 4 * TB * wave + 4 * lane;
+  f32x4 N[TB];
+  auto share = [&] {
+#pragma unroll
+    for (int t = 0; t < TB; ++t) {
+      quad_t q[NOPND];
+      split_quad(N[t], q);
+#pragma unroll
+      for (int o = 0; o < NOPND; ++o) sq[o][TB * wave + t][lane] = q[o];
+    }
+  };
+#pragma unroll
+  for (int t = 0; t < TB; ++t) N[t] = *(const f32x4*)(at + (c0 + 256 * t));
+  share();
+  for (int i = 1; i < nseg - 1; ++i) {
+    at += next;
+    const float* m = at + DK * p.dv;
+#pragma unroll
+    for (int t = 0; t < TB; ++t) N[t] = *(const f32x4*)(at + (c0 + 256 * t));
+    f32x4 a[TB][NS];
+#pragma unroll
+    for (int t = 0; t < TB; ++t)
+#pragma unroll
+      for (int k = 0; k < NS; ++k) a[t][k] = *(const f32x4*)(m + (uint32_t)((16 * (TB * wave + t) + l15) * DK + 16 * k + 4 * l4));
+    __syncthreads();
+#pragma unroll
+    for (int k = 0; k < NS; k += 2)
+#pragma unroll
+      for (int t = 0; t < TB; ++t) {
+        quad_t a0[NOPND], a1[NOPND];
+        split_quad(a[t][k], a0);
+        split_quad(a[t][k + 1], a1);
+#pragma unroll
+        for (int o = 0; o < NOPND; ++o) N[t] = mma_quads(a0[0], a1[0], sq[o][k][lane], sq[o][k + 1][lane], N[t]);
+        if constexpr (SPLIT) N[t] = mma_quads(a0[NOPND - 1], a1[NOPND - 1], sq[0][k][lane], sq[0][k + 1][lane], N[t]);
+      }
+    __syncthreads();
+#pragma unroll
+    for (int t = 0; t < TB; ++t) *(f32x4*)(at + (c0 + 256 * t)) = N[t];
+    share();
+  }
+}
+
 // ---- one token per sequence ----
 struct DeltaDecodeArgs {
   const elem_t* x; int64_t ld;
@@ -573,15 +612,18 @@ static int launch(const DeltaArgs& a, int segments, int multi, int n_chunks, hip
     case 4: hipLaunchKernelGGL(delta_conv_kernel<4>, cgrid, dim3(256), 0, s, a); break;
     default: hipLaunchKernelGGL(delta_conv_kernel<0>, cgrid, dim3(256), 0, s, a);
   }
-  hipLaunchKernelGGL((delta_chunk_kernel<DK>), dim3(n_chunks, a.H), dim3(64), 0, s, a);
+  hipLaunchKernelGGL((delta_chunk_kernel<DK>), dim3(a.H, n_chunks), dim3(64), 0, s, a);
   if (multi) {
     auto k = delta_prefill_kernel<DK, false>;
-    if (allow_lds(k, DeltaGeom<DK>::LDS)) return LM_EINVAL;
-    hipLaunchKernelGGL(k, dim3(segments, a.H, (a.dv + DK) / 64), dim3(256), DeltaGeom<DK>::LDS, s, a);
+    constexpr size_t lds = DeltaGeom<DK, false>::LDS;
+    if (allow_lds(k, lds)) return LM_EINVAL;
+    hipLaunchKernelGGL(k, dim3(segments, a.H, (a.dv + DK) / 64), dim3(256), lds, s, a);
+    hipLaunchKernelGGL(delta_chain_kernel<DK>, dim3(a.dv / 16, a.H, segments), dim3(256), 0, s, a);
   }
   auto k = delta_prefill_kernel<DK, true>;
-  if (allow_lds(k, DeltaGeom<DK>::LDS)) return LM_EINVAL;
-  hipLaunchKernelGGL(k, dim3(segments, a.H, a.dv / 64), dim3(256), DeltaGeom<DK>::LDS, s, a);
+  constexpr size_t lds = DeltaGeom<DK, true>::LDS;
+  if (allow_lds(k, lds)) return LM_EINVAL;
+  hipLaunchKernelGGL(k, dim3(segments, a.H, a.dv / 64), dim3(256), lds, s, a);
   return launch_status();
 }
 
@@ -597,7 +639,7 @@ extern "C" int lm_delta_prefill(const void* x, int64_t ld, void* o, int64_t ldo,
                                 const float* conv_w, int taps, float qk_eps, float scale,
                                 int64_t ab_col, const float* a_log, const float* dt_bias, void* y, float* norms, void* mats, float* vecs,
                                 int H, int G, int dk, int dv, void* stream) {
-  if (segments <= 0 || n_chunks < segments || (multi && !seg_state) || H <= 0 || G <= 0 || H % G || dv <= 0 || dv % 64 || taps <= 0 || ldo > (1 << 24) || ld % FR || ldo % 4 || !y ||
+  if (segments <= 0 || n_chunks > 65535 || n_chunks < segments || (multi && !seg_state) || H <= 0 || G <= 0 || H % G || dv <= 0 || dv % 64 || taps <= 0 || ldo > (1 << 24) || ld % FR || ldo % 4 || !y ||
       !norms || !mats || !vecs)
     return LM_EINVAL;
   DeltaArgs a{(const elem_t*)x, ld, (elem_t*)o, ldo, state, ring, portion, chunks, seg, seg_state, conv_w, taps, qk_eps, scale, ab_col, a_log, dt_bias,

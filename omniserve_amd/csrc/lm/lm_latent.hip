@@ -88,9 +88,9 @@ struct LatentDecodeArgs {
 template <int RP, int TP>
 struct LatentGeom {
   static constexpr int KT = 32, ROW = RP + TP, ES = (int)sizeof(elem_t);
-  static constexpr int CB = KT * RP * ES, TB = KT * TP * ES, BUF = CB + TB, QB = 16 * ROW * ES;
-  static constexpr int NBUF = 2 * BUF <= 155648 ? 2 : 1;
-  static constexpr size_t LDS = NBUF * BUF > QB ? NBUF * BUF : QB;
+  static constexpr int CB = KT * RP * ES, TB = KT * TP * ES, BUF = CB + TB;
+  static constexpr int NBUF = 2 * BUF <= 151552 ? 2 : 1;
+  static constexpr size_t LDS = NBUF * BUF;
 };
 
 template <int RP, int TP>
@@ -99,7 +99,8 @@ __global__ __launch_bounds__(256, SPLIT ? 2 : 1) void latent_decode_kernel(Laten
   typedef Tile<RP * (int)sizeof(elem_t)> CT;
   typedef Tile<TP * (int)sizeof(elem_t)> TT;
   constexpr int ROW = Gm::ROW, NCF = RP / KSTEP, NTF = TP / KSTEP, NVB = RP / 64;
-  extern __shared__ __attribute__((aligned(16))) uint8_t lds[];      // the queries, then the key tiles
+  extern __shared__ __attribute__((aligned(16))) uint8_t lds[];      // key tiles
+  __shared__ __attribute__((aligned(16))) elem_t qr[16][TP];
   __shared__ float red[4];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l15 = lane & 15, l4 = lane >> 4;
   const int b = blockIdx.x, h0 = 16 * blockIdx.y, nh = min(16, p.H - h0), split = blockIdx.z;
@@ -108,40 +109,6 @@ __global__ __launch_bounds__(256, SPLIT ? 2 : 1) void latent_decode_kernel(Laten
   const int nt = pos / Gm::KT + 1, per = (nt + p.nsplit - 1) / p.nsplit, ta = split * per, tb = min(nt, ta + per);
   const int* bt = p.bt + (int64_t)b * p.bt_stride;
   const elem_t* row = p.x + (int64_t)b * p.ld;
-
-  elem_t(*qs)[ROW] = (elem_t(*)[ROW])lds;
-  for (int i = tid; i < 16 * (RP / FR); i += 256) {
-    const int hh = i / (RP / FR), d = (i - hh * (RP / FR)) * FR;
-    *(frag_t*)&qs[hh][d] = hh < nh ? *(const frag_t*)(p.qa + ((int64_t)b * p.H + h0 + hh) * RP + d) : frag_t{};
-  }
-  for (int i = tid; i < 16 * (TP / 2); i += 256) {      // pairs; those past `half` are padding
-    const int hh = i / (TP / 2), d = i - hh * (TP / 2);
-    float a = 0.f, c = 0.f;
-    if (d < p.half && hh < nh) {
-      const elem_t* q = row + (int64_t)(h0 + hh) * p.dk + p.q_rot + d;
-      const float u = (float)q[0], v = (float)q[p.half];
-      float s, co;
-      sincosf((float)pos * p.freq[d], &s, &co);
-      a = u * co - v * s;
-      c = v * co + u * s;
-    }
-    const int at = d < p.half ? d : 2 * p.half + 2 * (d - p.half);
-    qs[hh][RP + at] = (elem_t)a;
-    qs[hh][RP + (d < p.half ? d + p.half : at + 1)] = (elem_t)c;
-  }
-  // the new row: written by every workgroup that reads it itself (equal bytes), the ones whose part holds the newest tile
-  const int slot = p.slot[b];
-  if (tb == nt && ta < tb && slot >= 0 && p.src_col >= 0)
-    latent_row(row + p.src_col, p.w, p.eps, p.freq, p.half, pos, p.cache + (int64_t)slot * ROW, p.R, RP, TP, red);
-  __syncthreads();      // (also makes the appended row visible to the other waves of this workgroup)
-  frag_t qf[NCF + NTF];
-#pragma unroll
-  for (int s = 0; s < NCF + NTF; ++s) qf[s] = *(const frag_t*)&qs[l15][s * KSTEP + FR * l4];
-  f32x4 acc[NVB];
-#pragma unroll
-  for (int c = 0; c < NVB; ++c) acc[c] = zero4();
-  float m_run = NEG, l_run = 0.f;
-  __syncthreads();      // the queries' place is free
 
   auto stage = [&](int t, uint8_t* buf) {
     const int kb = Gm::KT * t;
@@ -158,20 +125,59 @@ __global__ __launch_bounds__(256, SPLIT ? 2 : 1) void latent_decode_kernel(Laten
     }
   };
   static_assert(Gm::CB % 4096 == 0 && Gm::TB % 4096 == 0, "whole pieces for four waves");
+  // the new row: written by every workgroup that reads it itself (equal bytes), the ones whose part holds the newest tile
+  const int slot = p.slot[b];
+  if (tb == nt && ta < tb && slot >= 0 && p.src_col >= 0) {
+    latent_row(row + p.src_col, p.w, p.eps, p.freq, p.half, pos, p.cache + (int64_t)slot * ROW, p.R, RP, TP, red);
+    __syncthreads();    // (makes it visible to the other waves of this workgroup)
+  }
+  if (ta < tb) stage(ta, lds);
+  // queries: the latent part as it is, the turned part through LDS
+  frag_t qf[NCF + NTF];
+  const elem_t* qp = p.qa + ((int64_t)b * p.H + h0 + min(l15, nh - 1)) * RP + FR * l4;
+#pragma unroll
+  for (int s = 0; s < NCF; ++s) qf[s] = *(const frag_t*)(qp + s * KSTEP);
+  for (int i = tid; i < 16 * (TP / 2); i += 256) {      // pairs; those past `half` are padding
+    const int hh = i / (TP / 2), d = i - hh * (TP / 2);
+    float a = 0.f, c = 0.f;
+    if (d < p.half && hh < nh) {
+      const elem_t* q = row + (int64_t)(h0 + hh) * p.dk + p.q_rot + d;
+      const float u = (float)q[0], v = (float)q[p.half];
+      float s, co;
+      sincosf((float)pos * p.freq[d], &s, &co);
+      a = u * co - v * s;
+      c = v * co + u * s;
+    }
+    const int at = d < p.half ? d : 2 * p.half + 2 * (d - p.half);
+    qr[hh][at] = (elem_t)a;
+    qr[hh][d < p.half ? d + p.half : at + 1] = (elem_t)c;
+  }
+  f32x4 acc[NVB];
+#pragma unroll
+  for (int c = 0; c < NVB; ++c) acc[c] = zero4();
+  float m_run = NEG, l_run = 0.f;
   auto compute = [&](int t, const uint8_t* ct, auto prefetch) {
     const int kb = Gm::KT * t;
     const uint8_t* tt = ct + Gm::CB;
-    f32x4 x[2];
+    f32x4 x[2], y[2];                      // (two chains of products per block of keys)
+    x[0] = x[1] = y[0] = y[1] = zero4();
 #pragma unroll
-    for (int u = 0; u < 2; ++u) {
-      x[u] = zero4();
+    for (int s = 0; s < NCF; s += 2)
 #pragma unroll
-      for (int s = 0; s < NCF; ++s) x[u] = mma(CT::frag(ct, 16 * u + l15, 4 * s + l4), qf[s], x[u]);
+      for (int u = 0; u < 2; ++u) {
+        x[u] = mma(CT::frag(ct, 16 * u + l15, 4 * s + l4), qf[s], x[u]);
+        y[u] = mma(CT::frag(ct, 16 * u + l15, 4 * s + 4 + l4), qf[s + 1], y[u]);
+      }
 #pragma unroll
-      for (int s = 0; s < NTF; ++s) x[u] = mma(TT::frag(tt, 16 * u + l15, 4 * s + l4), qf[NCF + s], x[u]);
-      __builtin_amdgcn_sched_barrier(0);      // (not all of the tile's operands in registers at once)
-    }
-    prefetch();
+    for (int s = 0; s < NTF; s += 2)
+#pragma unroll
+      for (int u = 0; u < 2; ++u) {
+        x[u] = mma(TT::frag(tt, 16 * u + l15, 4 * s + l4), qf[NCF + s], x[u]);
+        y[u] = mma(TT::frag(tt, 16 * u + l15, 4 * s + 4 + l4), qf[NCF + s + 1], y[u]);
+      }
+#pragma unroll
+    for (int u = 0; u < 2; ++u) x[u] += y[u];
+    prefetch();                            // (behind the reads above: the compiler has the next LDS read wait for it)
     if (kb + Gm::KT - 1 > pos) {
 #pragma unroll
       for (int u = 0; u < 2; ++u)
@@ -188,19 +194,19 @@ __global__ __launch_bounds__(256, SPLIT ? 2 : 1) void latent_decode_kernel(Laten
       for (int o = 0; o < NOPND; ++o) acc[c] = mma_quads(v0, v1, pq[0][o], pq[1][o], acc[c]);
     }
   };
+  __syncthreads();
+#pragma unroll
+  for (int s = 0; s < NTF; ++s) qf[NCF + s] = *(const frag_t*)&qr[l15][s * KSTEP + FR * l4];
   if constexpr (Gm::NBUF == 2) {
-    if (ta < tb) stage(ta, lds);
-    __syncthreads();
     for (int t = ta; t < tb; ++t) {
-      uint8_t *now = lds + ((t - ta) & 1) * Gm::BUF, *next = lds + ((t - ta + 1) & 1) * Gm::BUF;
-      compute(t, now, [&] { if (t + 1 < tb) stage(t + 1, next); });
+      compute(t, lds + ((t - ta) & 1) * Gm::BUF, [&] { if (t + 1 < tb) stage(t + 1, lds + ((t - ta + 1) & 1) * Gm::BUF); });
       __syncthreads();
     }
   } else {
     for (int t = ta; t < tb; ++t) {
-      stage(t, lds);
-      __syncthreads();
       compute(t, lds, [] {});
+      __syncthreads();
+      if (t + 1 < tb) stage(t + 1, lds);
       __syncthreads();
     }
   }

@@ -438,8 +438,9 @@ class LatentAttention(Mixer):
         return ops.matmul(o, self.w_out)
 
     def splits(self, b) -> int:
-        """Parts of the keys per (sequence, 16 heads): enough workgroups for two per CU, at least 64 keys each."""
-        return max(1, min(512 // max(b.n_decode * ((self.s.heads + 15) // 16), 1), b.max_context // 64, 64))
+        """Parts of the keys per (sequence, 16 heads): two workgroups per CU if each gets 256 keys, else one, at least 64 keys each."""
+        groups = max(b.n_decode * ((self.s.heads + 15) // 16), 1)
+        return max(1, min(512 // groups, max(256 // groups, b.max_context // 256), b.max_context // 64, 64))
 
 
 class GatedLinearAttention(Mixer):
