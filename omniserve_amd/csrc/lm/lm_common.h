@@ -192,6 +192,21 @@ __device__ __forceinline__ void dma16(const void* src, void* lds_wave_base) {
                                    (__attribute__((address_space(3))) void*)lds_wave_base, 16, 0, 0);
 }
 
+// The same hidden from the compiler, which would wait for every DMA in flight in front of the next LDS read.  The kernel counts the
+// pieces itself (wait_pieces).  M0 is the compiler's: saved and restored.
+__device__ __forceinline__ void dma16_uncounted(const void* src, uint32_t lds_dst) {
+  uint32_t keep;
+  lds_dst = __builtin_amdgcn_readfirstlane(lds_dst);      // (uniform already; says so where the compiler cannot see it)
+  asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %2\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off\n\ts_mov_b32 m0, %0"
+               : "=&s"(keep)
+               : "v"(src), "s"(lds_dst)
+               : "memory");
+}
+template <int N>
+__device__ __forceinline__ void wait_pieces() {
+  asm volatile("s_waitcnt vmcnt(%0)" ::"n"(N) : "memory");
+}
+
 // Workgroups are dealt round-robin to the 8 XCDs: hands every XCD one contiguous range of [0, total).  The grid has
 // 8 * ceil(total / 8) workgroups; returns -1 for the surplus.
 __device__ __forceinline__ int xcd_contiguous(int wid, int total) {

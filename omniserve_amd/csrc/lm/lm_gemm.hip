@@ -203,20 +203,6 @@ __device__ __forceinline__ int stage_swizzle(int row) {
   return (((q ^ (q >> 1)) & 1) << 1) | (q >> 1);
 }
 
-// The LDS-DMA of a stage, hidden from the compiler: it would wait for every DMA in flight in front of the first LDS read.  The
-// loop counts the pieces itself (wait_pieces).  M0 is the compiler's: saved and restored.
-__device__ __forceinline__ void dma16_uncounted(const void* src, uint32_t lds_dst) {
-  uint32_t keep;
-  asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %2\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off\n\ts_mov_b32 m0, %0"
-               : "=&s"(keep)
-               : "v"(src), "s"(lds_dst)
-               : "memory");
-}
-template <int N>
-__device__ __forceinline__ void wait_pieces() {
-  asm volatile("s_waitcnt vmcnt(%0)" ::"n"(N) : "memory");
-}
-
 // 4 waves, 128 rows x 64 channels each; three stages: while one multiplies, two are on their way
 template <int EPI>
 __global__ __launch_bounds__(256, 2) void gemm_tiles_kernel(GemmArgs p, int mt_a, int mt_b) {

@@ -438,8 +438,8 @@ class LatentAttention(Mixer):
         return ops.matmul(o, self.w_out)
 
     def splits(self, b) -> int:
-        """Parts of the keys per (sequence, 16 heads): two workgroups per CU if each gets 256 keys, else one, at least 64 keys each."""
-        groups = max(b.n_decode * ((self.s.heads + 15) // 16), 1)
+        """Parts of the keys per (sequence, 32 heads): two workgroups per CU if each gets 256 keys, else one, at least 64 keys each."""
+        groups = max(b.n_decode * ((self.s.heads + 31) // 32), 1)
         return max(1, min(512 // groups, max(256 // groups, b.max_context // 256), b.max_context // 64, 64))
 
 
