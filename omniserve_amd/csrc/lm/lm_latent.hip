@@ -53,7 +53,22 @@ __global__ __launch_bounds__(256) void latent_append_kernel(LatentAppendArgs p) 
   }
   __syncthreads();
   elem_t* row = p.x + (int64_t)t * p.ld;
-  for (int i = tid; i < p.H * p.half; i += 256) {
+  if (p.half % 4 == 0 && p.q_rot % 4 == 0) {
+    const int nq = p.half / 4;
+    for (int i = tid; i < p.H * nq; i += 256) {
+      const int h = i / nq, d = 4 * (i - h * nq);
+      quad_t* q = (quad_t*)(row + (int64_t)h * p.dk + p.q_rot + d);
+      const f32x4 a = from_quad(q[0]), b = from_quad(q[nq]);
+      f32x4 u, v;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        u[e] = a[e] * cs[d + e][0] - b[e] * cs[d + e][1];
+        v[e] = b[e] * cs[d + e][0] + a[e] * cs[d + e][1];
+      }
+      q[0] = to_quad(u);
+      q[nq] = to_quad(v);
+    }
+  } else for (int i = tid; i < p.H * p.half; i += 256) {
     const int h = i / p.half, d = i - h * p.half;
     elem_t* q = row + (int64_t)h * p.dk + p.q_rot + d;
     const float a = (float)q[0], b = (float)q[p.half];

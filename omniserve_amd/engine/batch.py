@@ -47,14 +47,18 @@ class BatchBuilder:
     def __init__(self, model, device):
         self.page, self.attn_rows, self.device = model.page_size, model.attn_rows, device
         self.linear_wgs = model.linear_workgroups()
+        self.min_segments = model.min_segments
         self.chunk, self.expand = model.chunk_rows, model.expand_pages
 
     def _segment_len(self, portions: List[Entry]) -> int:
         """Tokens per segment of a recurrent layer: enough segments for two workgroups per CU, none below 256 tokens, at most 32
-        per portion (every segment starts from the sum of those before it)."""
+        per portion (every segment starts from the sum of those before it); none when the longest portion makes fewer than
+        min_segments (a first pass over the segments costs as much as it saves)."""
         total, longest = sum(len(e.tokens) for e in portions), max(len(e.tokens) for e in portions)
         want = max(1, 512 // max(self.linear_wgs, 1))
         n = max(256, -(-total // want), -(-longest // 32))
+        if longest < n * self.min_segments:
+            n = longest
         return -(-n // 64) * 64
 
     def build(self, entries: List[Entry]):

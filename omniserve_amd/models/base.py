@@ -11,6 +11,7 @@ class EngineModel:
 
     page_size = 64                       # tokens per cache page
     attn_rows = 128                      # query rows of one prefill attention tile
+    min_segments = 1                     # parts of a portion from which on recurrent layers run them in parallel
     chunk_rows = 0                       # tokens per chunk of recurrent layers that work in chunks (0: there are none)
     expand_pages = 0                     # most context pages a layer expands into keys and values at once (0: none does)
     dtypes: Tuple[torch.dtype, ...] = () # number formats the model runs in, its default first

@@ -438,9 +438,10 @@ class LatentAttention(Mixer):
         return ops.matmul(o, self.w_out)
 
     def splits(self, b) -> int:
-        """Parts of the keys per (sequence, 32 heads): two workgroups per CU if each gets 256 keys, else one, at least 64 keys each."""
-        groups = max(b.n_decode * ((self.s.heads + 31) // 32), 1)
-        return max(1, min(512 // groups, max(256 // groups, b.max_context // 256), b.max_context // 64, 64))
+        """Parts of the keys per (sequence, 32 heads): a workgroup per CU, two if each gets 1024 keys; at least 256 keys each (a part
+        leaves a latent of f32 per head)."""
+        groups, keys = max(b.n_decode * ((self.s.heads + 31) // 32), 1), b.max_context
+        return max(1, min(max(256 // groups, min(512 // groups, keys // 1024)), keys // 256, 64))
 
 
 class GatedLinearAttention(Mixer):
@@ -625,6 +626,7 @@ class Decoder(EngineModel):
         if len(shapes) > 1:
             raise ValueError("layers that mix values need the same kv heads and value size")
         kinds = {type(l.mixer) for l in self.layers}
+        self.min_segments = 3 if kinds & {GatedLinearAttention, DeltaRule} else 1
         self.chunk_rows = ops.delta_chunk if DeltaRule in kinds else 0
         self.expand_pages = EXPAND_PAGES if LatentAttention in kinds else 0
         self.tap = None          # called with the residual stream after every layer (tests); None in production
